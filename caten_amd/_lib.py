@@ -13,11 +13,12 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libcaten_hip.so")
 
 # constants of include/caten_hip.h
-F32, F16, Q4_0, Q8_0 = 0, 1, 2, 8
-GGML_TYPE = {"f32": F32, "f16": F16, "q4_0": Q4_0, "q8_0": Q8_0}
+F32, F16, Q4_0, Q8_0, BF16 = 0, 1, 2, 8, 30
+GGML_TYPE = {"f32": F32, "f16": F16, "q4_0": Q4_0, "q8_0": Q8_0, "bf16": BF16}
 PRO_NONE, PRO_LAYERNORM, PRO_RMSNORM, PRO_SWIGLU = 0, 1, 2, 3
 ACT_NONE, ACT_RELU, ACT_GELU, ACT_SILU, ACT_SIGMOID, ACT_TANH = 0, 1, 2, 3, 4, 5
-ARCH_GPT2, ARCH_LLAMA = 0, 1
+ARCH_GPT2, ARCH_LLAMA, ARCH_MIXED = 0, 1, 2
+MIXER_DELTA, MIXER_LATENT = 0, 1
 
 
 class HipError(RuntimeError):
@@ -32,6 +33,17 @@ class DecoderConfig(C.Structure):
     _fields_ = [("arch", C.c_int), ("n_layers", C.c_int), ("dim", C.c_int), ("n_heads", C.c_int),
                 ("n_kv_heads", C.c_int), ("ffn", C.c_int), ("vocab", C.c_int), ("max_seq", C.c_int),
                 ("eps", C.c_float), ("rope_base", C.c_float)]
+
+
+class LayerSpec(C.Structure):
+    _fields_ = [("mixer", C.c_int), ("heads", C.c_int), ("kv_heads", C.c_int), ("dim", C.c_int), ("vdim", C.c_int),
+                ("conv", C.c_int), ("kv_rank", C.c_int), ("scale", C.c_float), ("sink", C.c_int), ("gate", C.c_int),
+                ("ffn", C.c_int)]
+
+
+class MixedConfig(C.Structure):
+    _fields_ = [("n_layers", C.c_int), ("dim", C.c_int), ("vocab", C.c_int), ("max_seq", C.c_int), ("norm", C.c_int),
+                ("eps", C.c_float), ("position_base", C.c_float), ("logit_softcap", C.c_float), ("precision", C.c_int)]
 
 
 _vp, _vpp = C.c_void_p, C.POINTER(C.c_void_p)
@@ -107,10 +119,12 @@ PROTOTYPES = {
     "cthip_kv_append_paged": (_i, [_vp, _vp, _vp, _vp, _i, _i, _i]),
     "cthip_sdpa_cached_paged": (_i, [_vp, _vp, _vp, _vp, _i, _i, _i, _i]),
     "cthip_decoder_create": (_i, [_vpp, C.POINTER(DecoderConfig)]),
+    "cthip_decoder_create_mixed": (_i, [_vpp, C.POINTER(MixedConfig), C.POINTER(LayerSpec)]),
     "cthip_decoder_destroy": (_i, [_vp]),
     "cthip_decoder_load": (_i, [_vp, C.c_char_p, _i, _vp, _i64, _i64]),
     "cthip_decoder_missing": (_i, [_vp]),
     "cthip_decoder_forward": (_i, [_vp, _vp, _i, _i, C.POINTER(_i64), _vp]),
+    "cthip_decoder_forward_rows": (_i, [_vp, _vp, _i, _i, C.POINTER(_i), _i, C.POINTER(_i64), _vp]),
     "cthip_decoder_generate": (_i, [_vp, _i, _vp]),
     "cthip_decoder_generate_until": (_i, [_vp, _i, _i64, _vp, C.POINTER(_i)]),
     "cthip_decoder_position": (_i, [_vp]),

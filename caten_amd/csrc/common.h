@@ -74,9 +74,9 @@ int fail(int code, const char *fmt, ...);
 
 // ---- packed weight matrix ----
 struct WMat {
-  int type;         // CTHIP_F32 / F16 / Q4_0 / Q8_0
+  int type;         // CTHIP_F32 / F16 / BF16 / Q4_0 / Q8_0
   int64_t rows, cols;
-  void *q;          // quant plane: Q8_0 int8[rows][cols]; Q4_0 u8[rows][cols/2]; F32 float; F16 half
+  void *q;          // quant plane: Q8_0 int8[rows][cols]; Q4_0 u8[rows][cols/2]; F32 float; F16, BF16 16-bit floats
   void *d;          // scale plane: fp16[rows][cols/32] (quantised types), else NULL
   int64_t q_bytes, d_bytes;
   // the single-row kernels request this matrix with the non-temporal hint: set for a matrix that cannot stay in
@@ -159,6 +159,7 @@ struct GemvArgs {
   int pair_swiglu;
   int stage_x;  // set by the launcher: the workgroup stages the input vector in LDS once
   float eps;
+  float softcap;  // > 0: the stored value is softcap * tanh(value / softcap), before the argmax sees it
   int rows, cols;
   int act, pro;
   // A launch over a slice of the columns of a wider matrix (set by the launcher; 0 = the matrix is `cols` wide):
@@ -331,6 +332,8 @@ __device__ __forceinline__ float half_bits_to_float(unsigned short h) {
   return (float)__builtin_bit_cast(_Float16, h);
 }
 
+__device__ __forceinline__ float bf16_bits_to_float(unsigned short h) { return __uint_as_float((unsigned)h << 16); }
+
 // Caten's decompositions (api/function.lisp:437-440, nn/activations.lisp:3-7,202-215,
 // api/high-level-ops.lisp:112-117): exp(x) = exp2(x * 1/ln2); sigmoid = recip(1 + exp2(-x/ln2));
 // tanh(y) = 2*sigmoid(2y) - 1.
@@ -373,6 +376,8 @@ __device__ __forceinline__ float ct_gelu(float x) {
   const float u2 = -2.3022082f * (x * fmaf(0.044715f * x, x, 1.0f));  // -2 u log2(e)
   return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(u2));
 }
+// cap * tanh(x / cap)
+__device__ __forceinline__ float softcap(float x, float cap) { return cap * ct_tanh(x / cap); }
 __device__ __forceinline__ float ct_silu(float x) { return x * ct_sigmoid(x); }
 __device__ __forceinline__ float apply_act(int act, float v) {
   switch (act) {

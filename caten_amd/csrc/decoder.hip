@@ -21,6 +21,9 @@
 // run as one batch (MFMA GEMMs over the rows, see prefill()); shorter ones are fed row by row
 // through the decode step (causal attention makes that the same function).  Either way only the
 // last row runs lm_head and argmax.
+//
+// Decoders whose layers are listed one by one (CTHIP_ARCH_MIXED, not in the reference) share everything here but the
+// layers themselves (decoder_mixed.hip).
 #include <stdlib.h>
 #include <string.h>
 
@@ -30,102 +33,25 @@
 
 #include "common.h"
 #include "decode_fused.h"
+#include "decoder.h"
 
 namespace cthip {
-
-struct RawTensor {
-  void *dev = nullptr;  // GGUF bytes on the device
-  int type = 0;
-  int64_t rows = 0, cols = 0;
-  size_t nbytes = 0;
-};
 
 static size_t raw_nbytes(int type, int64_t n) {
   switch (type) {
     case CTHIP_F32: return (size_t)n * 4;
-    case CTHIP_F16: return (size_t)n * 2;
+    case CTHIP_F16: case CTHIP_BF16: return (size_t)n * 2;
     case CTHIP_Q8_0: return (size_t)((n + 31) / 32) * 34;
     case CTHIP_Q4_0: return (size_t)(n / 32) * 18;
     default: return 0;
   }
 }
 
-static const int kStepsPerGraph = 8;
-
-struct Layer {
-  // GPT-2
-  float *ln1_g = nullptr, *ln1_b = nullptr, *ln2_g = nullptr, *ln2_b = nullptr;
-  WMat *attn = nullptr, *proj = nullptr, *fc = nullptr, *fc2 = nullptr;
-  float *attn_b = nullptr, *proj_b = nullptr, *fc_b = nullptr, *fc2_b = nullptr;
-  // LayerNorm folded through c_attn / c_fc: S = W.gamma, C = W.beta + bias
-  float *attn_s = nullptr, *attn_c = nullptr, *fc_s = nullptr, *fc_c = nullptr;
-  // Llama: attn = wq|wk|wv, proj = wo, fc = gate|up, fc2 = down, ln1_g/ln2_g = rms weights
-  bool fc_pairs = false;  // gate / up rows interleaved, SwiGLU in the gate|up launch
-  float *k_cache = nullptr, *v_cache = nullptr;
-  // option kv_cache 1: the cache as Q8_0 rows instead (quant and scale planes; k_cache / v_cache stay null)
-  void *kq = nullptr, *kdq = nullptr, *vq = nullptr, *vdq = nullptr;
-  // option kv_cache 2: the cache in pages (kvp.hip): device tables of page pointers and the host's copy of them
-  float **k_pages = nullptr, **v_pages = nullptr;
-  std::vector<float *> k_page_host, v_page_host;
-  // three-launch decode layer: attn.c_proj by head and mlp.c_proj by 16-column slab (quant / scale planes)
-  void *proj_hq = nullptr, *proj_hd = nullptr, *fc2_sq = nullptr, *fc2_sd = nullptr;
-};
-
-struct Decoder {
-  cthip_decoder_config cfg;
-  std::map<std::string, RawTensor> raw;
-  std::vector<std::string> required;
-  bool finalized = false;
-  std::vector<Layer> layers;
-  float *wte = nullptr, *wpe = nullptr, *lnf_g = nullptr, *lnf_b = nullptr;
-  WMat *lm_head = nullptr;
-  float *lm_s = nullptr, *lm_c = nullptr;  // ln_f folded through lm_head
-  // activations
-  float *x = nullptr, *q = nullptr, *kv_tmp = nullptr, *att = nullptr, *h = nullptr, *logits = nullptr;
-  AttnSplit att_split = {1, nullptr, nullptr};  // the one-launch-per-Linear step: workgroups per head of its attention launch
-  // device-resident loop state: [0] = current token, [1] = position
-  int *tokpos = nullptr;
-  int64_t *token64 = nullptr;
-  int64_t *history = nullptr;
-  int *hist_n = nullptr;
-  int *ctrl = nullptr;        // [0] = token id that ends a sequence (-1 = none), [1] = the sequence has ended
-  int *ctrl_host = nullptr;   // pinned copy of ctrl the host polls between graph launches
-  hipEvent_t ctrl_ev = nullptr;
-  // scratch of the argmax fused behind lm_head: one partial per wavefront
-  float *am_val = nullptr;
-  int *am_idx = nullptr;
-  int position = 0;
-  bool primed = false;  // a forward has left token/position on the device
-  bool use_graph = true;
-  // the three-launch decode layer (decode_fused.hip): second residual buffer, per-head partials of the
-  // attention projection, per-XCD accumulators of the MLP projection
-  bool fused = false;
-  float *x2 = nullptr, *patt = nullptr;
-  long long *pmlp = nullptr;
-  // all layers of a step as one launch (decode_flow.hip): the tagged hand-over buffers and the launch's arguments
-  bool flow = false;
-  FlowArgs flow_args = {};
-  // grouped-query layers (decode_gqa.hip): the attention projection has an accumulator set of its own
-  bool fused_gqa = false;
-  long long *pattn = nullptr;
-  // KV cache kept as Q8_0 rows (kvq.hip); peek_f32: fp32 copy of one layer's cache for cthip_decoder_peek
-  bool kvq = false;
-  float *peek_f32 = nullptr;
-  // KV cache in pages (kvp.hip)
-  bool kvp = false;
-  // [0]: the step as the session runs it at short contexts; [1]: three-launch layers at long contexts (long_from > 0):
-  // the attention as a launch of its own with a head's keys shared by several workgroups, then the projection
-  hipGraphExec_t g_step[2] = {nullptr, nullptr}, g_body[2] = {nullptr, nullptr}, g_multi[2] = {nullptr, nullptr};
-  int long_from = 0;       // position from which [1] runs; 0 = never
-  bool long_mode = false;  // which of the two queue_step queues
-  int64_t weight_bytes = 0, vector_bytes = 0;
-  std::vector<void *> owned;  // device blocks to free
-};
-
 static int kv_dim(const cthip_decoder_config &c) { return c.dim / c.n_heads * c.n_kv_heads; }
 
 static void build_required(Decoder *d) {
   const cthip_decoder_config &c = d->cfg;
+  if (c.arch == CTHIP_ARCH_MIXED) return mixed_required(d);
   char buf[128];
   if (c.arch == CTHIP_ARCH_GPT2) {
     // state-dict keys after remap-key (apps/gpt2/gpt2.lisp:52-70)
@@ -151,14 +77,14 @@ static void build_required(Decoder *d) {
   }
 }
 
-static int dev_alloc(Decoder *d, void **p, size_t bytes) {
+int dev_alloc(Decoder *d, void **p, size_t bytes) {
   int rc = cthip_alloc(p, bytes);
   if (rc == 0) d->owned.push_back(*p);
   return rc;
 }
 
 // dequantise a raw tensor to an fp32 device vector owned by the session
-static int to_f32(Decoder *d, const std::string &key, int64_t want_n, float **out) {
+int to_f32(Decoder *d, const std::string &key, int64_t want_n, float **out) {
   auto it = d->raw.find(key);
   if (it == d->raw.end()) return fail(CTHIP_E_STATE, "decoder: tensor '%s' was not loaded", key.c_str());
   RawTensor &r = it->second;
@@ -176,8 +102,7 @@ static int to_f32(Decoder *d, const std::string &key, int64_t want_n, float **ou
 
 // pack one or more raw tensors (row-concatenated) into a weight matrix
 // interleave: two parts of equal height are merged row by row (a0, b0, a1, b1, ...) instead of stacked
-static int to_wmat(Decoder *d, const std::vector<std::string> &keys, int64_t want_rows, int64_t want_cols, WMat **out,
-                   bool interleave = false) {
+int to_wmat(Decoder *d, const std::vector<std::string> &keys, int64_t want_rows, int64_t want_cols, WMat **out, bool interleave) {
   std::vector<RawTensor *> parts;
   int64_t rows = 0;
   for (const std::string &k : keys) {
@@ -252,18 +177,18 @@ static int ensure_pages(Decoder *d, int rows) {
 static int queue_step(Decoder *d, bool with_head, bool embed = true);
 static int queue_head(Decoder *d);
 
-// S = W.gamma and C = W.beta + bias for a LayerNorm that precedes the Linear W
-static int make_fold(Decoder *d, const WMat *w, const float *gamma, const float *beta, const float *bias, float **S,
-                     float **C) {
+// S = W.gamma and C = W.beta + bias for a LayerNorm that precedes the Linear W (beta null: S only)
+int make_fold(Decoder *d, const WMat *w, const float *gamma, const float *beta, const float *bias, float **S, float **C) {
   int rc;
   if ((rc = dev_alloc(d, (void **)S, sizeof(float) * (size_t)w->rows))) return rc;
-  if ((rc = dev_alloc(d, (void **)C, sizeof(float) * (size_t)w->rows))) return rc;
   GemvArgs a = {};
   a.x = gamma;
   a.y = *S;
   a.x_stride = w->cols;
   a.y_stride = w->rows;
   if ((rc = launch_gemv(w, a, 1))) return rc;
+  if (!beta) return 0;
+  if ((rc = dev_alloc(d, (void **)C, sizeof(float) * (size_t)w->rows))) return rc;
   GemvArgs b = {};
   b.x = beta;
   b.bias = bias;
@@ -281,7 +206,8 @@ static int finalize(Decoder *d) {
   const int D = c.dim, F = c.ffn, V = c.vocab, KD = kv_dim(c);
   int rc;
   char b[128];
-  d->layers.resize(c.n_layers);
+  const bool mixed = c.arch == CTHIP_ARCH_MIXED;
+  if (!mixed) d->layers.resize(c.n_layers);
   auto key = [&](int l, const char *s) {
     snprintf(b, sizeof(b), c.arch == CTHIP_ARCH_GPT2 ? "h.%d.%s" : "layers.%d.%s", l, s);
     return std::string(b);
@@ -290,7 +216,9 @@ static int finalize(Decoder *d) {
   do {                         \
     if ((rc = (e))) return rc; \
   } while (0)
-  if (c.arch == CTHIP_ARCH_GPT2) {
+  if (mixed) {
+    TRY(mixed_load(d));
+  } else if (c.arch == CTHIP_ARCH_GPT2) {
     TRY(to_f32(d, "wte.weight", (int64_t)V * D, &d->wte));
     TRY(to_f32(d, "wpe.weight", (int64_t)c.max_seq * D, &d->wpe));
     TRY(to_f32(d, "ln_f.affine", D, &d->lnf_g));
@@ -339,11 +267,12 @@ static int finalize(Decoder *d) {
   d->vector_bytes -= 4 * (int64_t)V * D;
   if (c.arch == CTHIP_ARCH_GPT2) d->vector_bytes -= 4 * (int64_t)c.max_seq * D;
 
+  if (mixed && state().kv_cache) return fail(CTHIP_E_UNSUPPORTED, "decoder: a mixed decoder keeps its latents as fp32 rows (option kv_cache 0)");
   d->kvq = state().kv_cache == 1;
   d->kvp = state().kv_cache == 2;
   if (d->kvq && KD % 32) return fail(CTHIP_E_UNSUPPORTED, "decoder: a Q8_0 KV cache needs rows of whole 32-element blocks, not %d", KD);
   if (d->kvp && KD % 4) return fail(CTHIP_E_UNSUPPORTED, "decoder: a paged KV cache needs rows of a multiple of four floats, not %d", KD);
-  for (int l = 0; l < c.n_layers; l++) {
+  for (int l = 0; l < c.n_layers && !mixed; l++) {
     Layer &L = d->layers[l];
     if (d->kvp) {  // tables of page pointers, all null: pages are opened as positions are reached (ensure_pages)
       const size_t np = (size_t)(c.max_seq + kKvPageRows - 1) / kKvPageRows;
@@ -364,10 +293,11 @@ static int finalize(Decoder *d) {
   }
   const int hdim = c.arch == CTHIP_ARCH_GPT2 ? F : 2 * F;
   TRY(dev_alloc(d, (void **)&d->x, sizeof(float) * D));
-  TRY(dev_alloc(d, (void **)&d->q, sizeof(float) * D));
-  TRY(dev_alloc(d, (void **)&d->kv_tmp, sizeof(float) * 2 * KD));
-  TRY(dev_alloc(d, (void **)&d->att, sizeof(float) * D));
-  {
+  if (!mixed) {
+    TRY(dev_alloc(d, (void **)&d->q, sizeof(float) * D));
+    TRY(dev_alloc(d, (void **)&d->kv_tmp, sizeof(float) * 2 * KD));
+    TRY(dev_alloc(d, (void **)&d->att, sizeof(float) * D));
+    TRY(dev_alloc(d, (void **)&d->h, sizeof(float) * hdim));
     // long contexts: the keys of a head shared by as many workgroups as give every compute unit one (at most 16):
     // all of a launch's workgroups are then resident together and ask for their rows at once
     const int Dh = D / c.n_heads;
@@ -380,7 +310,6 @@ static int finalize(Decoder *d) {
       d->att_split.ranges = ranges;
     }
   }
-  TRY(dev_alloc(d, (void **)&d->h, sizeof(float) * hdim));
   TRY(dev_alloc(d, (void **)&d->logits, sizeof(float) * V));
   TRY(dev_alloc(d, (void **)&d->tokpos, 256));
   TRY(dev_alloc(d, (void **)&d->token64, 256));
@@ -402,6 +331,7 @@ static int finalize(Decoder *d) {
     // non-temporally and stops evicting what the step does reuse.
     std::vector<WMat *> ws = {d->lm_head};
     for (Layer &L : d->layers) ws.insert(ws.end(), {L.attn, L.proj, L.fc, L.fc2});
+    for (MixedLayer &L : d->mixed) ws.insert(ws.end(), {L.in, L.out, L.gate_up, L.down});
     int64_t total = 0;
     for (WMat *w : ws) total += w ? w->q_bytes + w->d_bytes : 0;
     for (WMat *w : ws)
@@ -574,7 +504,12 @@ static int queue_step(Decoder *d, bool with_head, bool embed) {
   } while (0)
   const bool gpt2 = c.arch == CTHIP_ARCH_GPT2;
   // embed = false: the previous step's head has already gathered this step's input (queue_head)
-  if (embed) TRY(launch_embedding(d->x, d->wte, nullptr, tok, 1, V, D, gpt2 ? d->wpe : nullptr, pos, c.max_seq));
+  if (embed) TRY(launch_embedding(d->x, d->wte, nullptr, tok, 1, V, D, d->wpe, pos, c.max_seq));
+  if (c.arch == CTHIP_ARCH_MIXED) {
+    TRY(mixed_queue_layers(d));
+    if (with_head) TRY(queue_head(d));
+    return 0;
+  }
   if (d->flow) {
     TRY(launch_dec_flow(d->flow_args));
     if (with_head) TRY(queue_head(d));
@@ -832,10 +767,11 @@ static int queue_step(Decoder *d, bool with_head, bool embed) {
 // ln_f -> lm_head GEMV on d->x, greedy token -> tokpos[0] and the history, position + 1
 static int queue_head(Decoder *d) {
   const cthip_decoder_config &c = d->cfg;
-  const bool gpt2 = c.arch == CTHIP_ARCH_GPT2;
+  const bool layernorm = c.arch == CTHIP_ARCH_GPT2 || (c.arch == CTHIP_ARCH_MIXED && d->mcfg.norm == CTHIP_PRO_LAYERNORM);
   GemvArgs o = {};
   o.x = d->x;
-  o.pro = gpt2 ? CTHIP_PRO_LAYERNORM : CTHIP_PRO_RMSNORM;
+  o.pro = layernorm ? CTHIP_PRO_LAYERNORM : CTHIP_PRO_RMSNORM;
+  o.softcap = d->mcfg.logit_softcap;
   o.norm_g = d->lnf_g;
   o.norm_b = d->lnf_b;
   o.eps = c.eps;
@@ -857,7 +793,7 @@ static int queue_head(Decoder *d) {
   // ... and its embedding rows become the next step's input, in the block that settles the token
   o.nx_out = d->x;
   o.nx_wte = d->wte;
-  o.nx_wpe = gpt2 ? d->wpe : nullptr;
+  o.nx_wpe = d->wpe;
   o.nx_dim = c.dim;
   o.nx_vocab = c.vocab;
   o.nx_max_pos = c.max_seq;
@@ -868,12 +804,76 @@ static int queue_head(Decoder *d) {
 // an MFMA GEMM over the s rows (weights dequantised while staged), attention runs all s query rows
 // against the cache under the causal mask; only the last row goes through lm_head.
 static const int kPrefillMin = 8;
-static int prefill(Decoder *d, const int *ids, int s, int n) {
+
+int linear_residual_norm(float *XN, float *X, const WMat *w, const float *in, int s, int D, const float *bias, const float *g,
+                         const float *b, float eps, bool rms, int precision) {
+  auto norm = [&]() { return rms ? cthip_rmsnorm(XN, X, g, eps, s, D) : cthip_layernorm(XN, X, g, b, eps, s, D); };
+  GemmDeferred df;
+  const bool fuse = g != nullptr && reduce_norm_supported(D, 1);
+  int r = launch_linear_gemm(X, w, in, s, bias, X, CTHIP_ACT_NONE, precision, fuse ? &df : nullptr);
+  if (r) return r;
+  if (df.ws) {
+    if (reduce_norm_supported(D, df.ksplit)) {
+      r = launch_reduce_norm(XN, X, df.ws, df.ksplit, (int64_t)s * D, bias, X, g, b, eps, s, D, rms);
+    } else {  // too many shares of too wide a row to hold at once: reduce, then normalise
+      r = launch_splitk_reduce(X, df.ws, df.ksplit, s, D, bias, X);
+      if (!r) r = norm();
+    }
+    const int r2 = cthip_free(df.ws);  // stream-ordered: reused only by later work on this stream
+    return r ? r : r2;
+  }
+  return g ? norm() : 0;
+}
+
+// logits of `n_rows` rows of X (s, dim), the residual stream behind the last layer -> host
+static int score_rows(Decoder *d, const float *X, const int *rows, int n_rows, int precision, float *logits_out) {
+  const cthip_decoder_config &c = d->cfg;
+  const int D = c.dim, V = c.vocab;
+  const bool rms = c.arch == CTHIP_ARCH_LLAMA || (c.arch == CTHIP_ARCH_MIXED && d->mcfg.norm == CTHIP_PRO_RMSNORM);
+  const int kBatch = 256;  // rows at a time
+  float *A = nullptr, *B = nullptr, *Lg = nullptr;
+  int *idx = nullptr, rc = 0;
+  const int most = n_rows < kBatch ? n_rows : kBatch;
+#define TRY(e)                 \
+  do {                         \
+    if ((rc = (e))) goto done; \
+  } while (0)
+  TRY(alloc_scratch((void **)&A, sizeof(float) * (size_t)most * D));
+  TRY(alloc_scratch((void **)&B, sizeof(float) * (size_t)most * D));
+  TRY(alloc_scratch((void **)&Lg, sizeof(float) * (size_t)most * V));
+  TRY(alloc_scratch((void **)&idx, sizeof(int) * (size_t)most));
+  for (int r0 = 0; r0 < n_rows; r0 += kBatch) {
+    const int m = n_rows - r0 < kBatch ? n_rows - r0 : kBatch;
+    TRY(cthip_h2d(idx, rows + r0, sizeof(int) * (size_t)m));
+    TRY(launch_gather_rows(A, X, idx, m, D));
+    TRY(rms ? cthip_rmsnorm(B, A, d->lnf_g, c.eps, m, D) : cthip_layernorm(B, A, d->lnf_g, d->lnf_b, c.eps, m, D));
+    if (m >= kPrefillMin) {
+      TRY(launch_linear_gemm(Lg, d->lm_head, B, m, nullptr, nullptr, CTHIP_ACT_NONE, precision));
+    } else {
+      GemvArgs o = {};
+      o.x = B;
+      o.y = Lg;
+      o.x_stride = D;
+      o.y_stride = V;
+      TRY(launch_gemv(d->lm_head, o, m));
+    }
+    if (d->mcfg.logit_softcap > 0.0f) TRY(launch_softcap(Lg, (int64_t)m * V, d->mcfg.logit_softcap));
+    TRY(cthip_d2h(logits_out + (size_t)r0 * V, Lg, sizeof(float) * (size_t)m * V));
+  }
+#undef TRY
+done:
+  for (void *p : {(void *)A, (void *)B, (void *)Lg, (void *)idx})
+    if (p) cthip_free(p);
+  return rc;
+}
+
+static int prefill(Decoder *d, const int *ids, int s, int n, const int *rows, int n_rows, float *rows_out) {
   const cthip_decoder_config &c = d->cfg;
   const bool gpt2 = c.arch == CTHIP_ARCH_GPT2;
   const int D = c.dim, F = c.ffn, V = c.vocab, KD = kv_dim(c), Dh = c.dim / c.n_heads;
+  const bool mixed = c.arch == CTHIP_ARCH_MIXED;
   const int QW = D + 2 * KD, HW = gpt2 ? F : 2 * F;
-  const int prec = state().gemm_precision;
+  const int prec = mixed && d->mcfg.precision >= 0 ? d->mcfg.precision : state().gemm_precision;
   int rc = 0;
   float *X = nullptr, *XN = nullptr, *QKV = nullptr, *Q = nullptr, *ATT = nullptr, *Hb = nullptr, *G = nullptr, *KF = nullptr, *VF = nullptr;
   int *ids_dev = nullptr;
@@ -889,11 +889,13 @@ static int prefill(Decoder *d, const int *ids, int s, int n) {
   } while (0)
   TRY(alloc((void **)&X, sizeof(float) * (size_t)s * D));
   TRY(alloc((void **)&XN, sizeof(float) * (size_t)s * D));
-  TRY(alloc((void **)&QKV, sizeof(float) * (size_t)s * QW));
-  TRY(alloc((void **)&Q, sizeof(float) * (size_t)s * D));
-  TRY(alloc((void **)&ATT, sizeof(float) * (size_t)s * D));
-  TRY(alloc((void **)&Hb, sizeof(float) * (size_t)s * HW));
-  if (!gpt2) TRY(alloc((void **)&G, sizeof(float) * (size_t)s * F));
+  if (!mixed) {
+    TRY(alloc((void **)&QKV, sizeof(float) * (size_t)s * QW));
+    TRY(alloc((void **)&Q, sizeof(float) * (size_t)s * D));
+    TRY(alloc((void **)&ATT, sizeof(float) * (size_t)s * D));
+    TRY(alloc((void **)&Hb, sizeof(float) * (size_t)s * HW));
+  }
+  if (!gpt2 && !mixed) TRY(alloc((void **)&G, sizeof(float) * (size_t)s * F));
   if (d->kvq || d->kvp) {
     TRY(alloc((void **)&KF, sizeof(float) * (size_t)(n + s) * KD));
     TRY(alloc((void **)&VF, sizeof(float) * (size_t)(n + s) * KD));
@@ -904,31 +906,18 @@ static int prefill(Decoder *d, const int *ids, int s, int n) {
     int tp[2] = {ids[s - 1], n};  // position base for the learned position rows
     TRY(cthip_h2d(d->tokpos, tp, sizeof(tp)));
   }
-  TRY(launch_embedding(X, d->wte, nullptr, ids_dev, s, V, D, gpt2 ? d->wpe : nullptr, d->tokpos + 1, c.max_seq));
-  {
+  TRY(launch_embedding(X, d->wte, nullptr, ids_dev, s, V, D, d->wpe, d->tokpos + 1, c.max_seq));
+  if (mixed) {
+    TRY(mixed_prefill(d, X, XN, s, n));
+  } else {
     // A row-split Linear (attention projection, second MLP Linear) whose reduction axis was shared among several
     // workgroups per tile leaves partial tiles; what follows it is the residual add and the next norm, so one pass
     // over the rows does all three (launch_reduce_norm) instead of a reduction launch and a norm launch.
     auto norm = [&](float *y, const float *x, const float *g, const float *b) {
       return gpt2 ? cthip_layernorm(y, x, g, b, c.eps, s, D) : cthip_rmsnorm(y, x, g, c.eps, s, D);
     };
-    // X += W.in + bias, then XN = norm(X) with (g, b); g == nullptr: no norm follows (after the last layer)
-    auto linear_residual_norm = [&](const WMat *w, const float *in, const float *bias, const float *g, const float *b) {
-      GemmDeferred df;
-      const bool fuse = g != nullptr && reduce_norm_supported(D, 1);
-      int r = launch_linear_gemm(X, w, in, s, bias, X, CTHIP_ACT_NONE, prec, fuse ? &df : nullptr);
-      if (r) return r;
-      if (df.ws) {
-        if (reduce_norm_supported(D, df.ksplit)) {
-          r = launch_reduce_norm(XN, X, df.ws, df.ksplit, (int64_t)s * D, bias, X, g, b, c.eps, s, D, !gpt2);
-        } else {  // too many shares of too wide a row to hold at once: reduce, then normalise
-          r = launch_splitk_reduce(X, df.ws, df.ksplit, s, D, bias, X);
-          if (!r) r = norm(XN, X, g, b);
-        }
-        const int r2 = cthip_free(df.ws);  // stream-ordered: reused only by later work on this stream
-        return r ? r : r2;
-      }
-      return g ? norm(XN, X, g, b) : 0;
+    auto residual_norm = [&](const WMat *w, const float *in, const float *bias, const float *g, const float *b) {
+      return linear_residual_norm(XN, X, w, in, s, D, bias, g, b, c.eps, !gpt2, prec);
     };
     TRY(norm(XN, X, d->layers[0].ln1_g, d->layers[0].ln1_b));
     for (int l = 0; l < c.n_layers; l++) {
@@ -963,7 +952,7 @@ static int prefill(Decoder *d, const int *ids, int s, int n) {
       }
       TRY(launch_attn(ATT, Q, L.k_cache, L.v_cache, s, n, nullptr, n + s, c.n_heads, c.n_kv_heads, Dh));
       }
-      TRY(linear_residual_norm(L.proj, ATT, L.proj_b, L.ln2_g, L.ln2_b));
+      TRY(residual_norm(L.proj, ATT, L.proj_b, L.ln2_g, L.ln2_b));
       const float *hin = Hb;
       if (!gpt2 && L.fc_pairs && (2 * F) % 4 == 0) {  // SwiGLU in the epilogue of the gate|up launch
         TRY(launch_linear_gemm(G, L.fc, XN, s, L.fc_b, nullptr, kActSwigluPairs, prec));
@@ -977,9 +966,10 @@ static int prefill(Decoder *d, const int *ids, int s, int n) {
         }
       }
       const bool last = l + 1 == c.n_layers;
-      TRY(linear_residual_norm(L.fc2, hin, L.fc2_b, last ? nullptr : d->layers[l + 1].ln1_g, last ? nullptr : d->layers[l + 1].ln1_b));
+      TRY(residual_norm(L.fc2, hin, L.fc2_b, last ? nullptr : d->layers[l + 1].ln1_g, last ? nullptr : d->layers[l + 1].ln1_b));
     }
   }
+  if (n_rows > 0) TRY(score_rows(d, X, rows, n_rows, prec, rows_out));
   // the last row continues through the decode-step head
   TRY(cthip_d2d(d->x, X + (size_t)(s - 1) * D, sizeof(float) * D));
   {
@@ -1030,7 +1020,7 @@ int cthip_decoder_create(void **dec, const cthip_decoder_config *cfg) {
   CTHIP_REQUIRE_INIT();
   CTHIP_ARG(dec != nullptr && cfg != nullptr);
   const cthip_decoder_config &c = *cfg;
-  CTHIP_ARG(c.arch == CTHIP_ARCH_GPT2 || c.arch == CTHIP_ARCH_LLAMA);
+  CTHIP_ARG(c.arch == CTHIP_ARCH_GPT2 || c.arch == CTHIP_ARCH_LLAMA);  // (mixed decoders: cthip_decoder_create_mixed)
   CTHIP_ARG(c.n_layers > 0 && c.dim > 0 && c.n_heads > 0 && c.ffn > 0 && c.vocab > 0 && c.max_seq > 0);
   CTHIP_ARG(c.dim % c.n_heads == 0);
   CTHIP_ARG(c.n_kv_heads > 0 && c.n_heads % c.n_kv_heads == 0);
@@ -1042,6 +1032,44 @@ int cthip_decoder_create(void **dec, const cthip_decoder_config *cfg) {
   if (c.max_seq > 8192) return fail(CTHIP_E_UNSUPPORTED, "cthip_decoder_create: max_seq %d > 8192", c.max_seq);
   Decoder *d = new Decoder();
   d->cfg = c;
+  build_required(d);
+  *dec = d;
+  return 0;
+}
+
+int cthip_decoder_create_mixed(void **dec, const cthip_mixed_config *cfg, const cthip_layer_spec *layers) {
+  CTHIP_REQUIRE_INIT();
+  CTHIP_ARG(dec != nullptr && cfg != nullptr && layers != nullptr);
+  const cthip_mixed_config &c = *cfg;
+  CTHIP_ARG(c.n_layers > 0 && c.dim > 0 && c.vocab > 0 && c.max_seq > 0);
+  CTHIP_ARG(c.norm == CTHIP_PRO_LAYERNORM || c.norm == CTHIP_PRO_RMSNORM);
+  CTHIP_ARG(c.precision >= -1 && c.precision <= GEMM_BF16X6);
+  CTHIP_ARG(c.logit_softcap >= 0.0f && c.position_base >= 0.0f);
+  for (int l = 0; l < c.n_layers; l++) {
+    const cthip_layer_spec &s = layers[l];
+    CTHIP_ARG(s.mixer == CTHIP_MIXER_DELTA || s.mixer == CTHIP_MIXER_LATENT);
+    CTHIP_ARG(s.heads > 0 && s.dim > 0 && s.vdim > 0 && s.ffn >= 0);
+    if (s.dim > 256 || s.vdim > 256)
+      return fail(CTHIP_E_UNSUPPORTED, "cthip_decoder_create_mixed: layer %d: heads of %d / %d (at most 256)", l, s.dim, s.vdim);
+    if (s.mixer == CTHIP_MIXER_DELTA) {
+      CTHIP_ARG(s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.conv > 0);
+    } else {
+      CTHIP_ARG(s.kv_rank > 0);
+      if (s.kv_rank > 1024) return fail(CTHIP_E_UNSUPPORTED, "cthip_decoder_create_mixed: layer %d: a latent of %d (at most 1024)", l, s.kv_rank);
+    }
+  }
+  Decoder *d = new Decoder();
+  d->mcfg = c;
+  d->cfg = {};
+  d->cfg.arch = CTHIP_ARCH_MIXED;
+  d->cfg.n_layers = c.n_layers;
+  d->cfg.dim = c.dim;
+  d->cfg.n_heads = d->cfg.n_kv_heads = 1;
+  d->cfg.vocab = c.vocab;
+  d->cfg.max_seq = c.max_seq;
+  d->cfg.eps = c.eps;
+  d->mixed.resize(c.n_layers);
+  for (int l = 0; l < c.n_layers; l++) d->mixed[l].sp = layers[l];
   build_required(d);
   *dec = d;
   return 0;
@@ -1066,6 +1094,7 @@ int cthip_decoder_destroy(void *dec) {
     cthip_wmat_destroy(L.fc);
     cthip_wmat_destroy(L.fc2);
   }
+  mixed_release(d);
   cthip_wmat_destroy(d->lm_head);
   delete d;
   return 0;
@@ -1112,10 +1141,8 @@ int cthip_decoder_missing(const void *dec) {
   return n;
 }
 
-int cthip_decoder_forward(void *dec, const float *tokens, int s, int n, int64_t *token, float *logits_out) {
-  CTHIP_REQUIRE_INIT();
-  CTHIP_ARG(dec != nullptr && tokens != nullptr && token != nullptr);
-  Decoder *d = (Decoder *)dec;
+// logits_out: the last position's (rows null) or those of the `n_rows` listed ones
+static int forward_impl(Decoder *d, const float *tokens, int s, int n, const int *rows, int n_rows, int64_t *token, float *logits_out) {
   const cthip_decoder_config &c = d->cfg;
   if (s < 1) return fail(CTHIP_E_BAD_ARG, "cthip_decoder_forward: s = %d; a forward needs at least one token", s);
   if (n < 0 || n + s > c.max_seq)
@@ -1123,6 +1150,13 @@ int cthip_decoder_forward(void *dec, const float *tokens, int s, int n, int64_t 
                 n + s - 1, c.max_seq);
   int rc = finalize(d);
   if (rc) return rc;
+  if (c.arch == CTHIP_ARCH_MIXED) {
+    // the recurrent state holds the tokens before `position` and cannot go back
+    if (n != 0 && (!d->primed || n != d->position))
+      return fail(CTHIP_E_BAD_ARG, "cthip_decoder_forward: this decoder's state is at position %d; a forward starts there or at 0, not at %d",
+                  d->primed ? d->position : 0, n);
+    d->primed = false;  // until this forward is complete
+  }
   if ((rc = ensure_pages(d, n + s))) return rc;
   int zero = 0;
   if ((rc = cthip_h2d(d->hist_n, &zero, sizeof(int)))) return rc;
@@ -1137,20 +1171,41 @@ int cthip_decoder_forward(void *dec, const float *tokens, int s, int n, int64_t 
     ids[i] = (tf >= 0.0f && tf < (float)c.vocab && (float)(int)tf == tf) ? (int)tf : -1;
   }
   if (s >= kPrefillMin && state().prefill_gemm) {
-    if ((rc = prefill(d, ids.data(), s, n))) return rc;
+    if ((rc = prefill(d, ids.data(), s, n, rows, n_rows, logits_out))) return rc;
   } else {
     for (int i = 0; i < s; i++) {
       int tp[2] = {ids[i], n + i};
       if ((rc = cthip_h2d(d->tokpos, tp, sizeof(tp)))) return rc;
-      if ((rc = run_step(d, i == s - 1, n + i))) return rc;
+      bool wanted = false;
+      for (int r = 0; r < n_rows; r++) wanted |= rows[r] == i;
+      if ((rc = run_step(d, wanted || i == s - 1, n + i))) return rc;
+      for (int r = 0; r < n_rows; r++)
+        if (rows[r] == i && (rc = cthip_d2h(logits_out + (size_t)r * c.vocab, d->logits, sizeof(float) * (size_t)c.vocab))) return rc;
     }
   }
-  if (logits_out && (rc = cthip_d2h(logits_out, d->logits, sizeof(float) * (size_t)c.vocab))) return rc;
+  if (!rows && logits_out && (rc = cthip_d2h(logits_out, d->logits, sizeof(float) * (size_t)c.vocab))) return rc;
   if ((rc = cthip_d2h(token, d->token64, sizeof(int64_t)))) return rc;
   if ((rc = flow_check(d))) return rc;
   d->position = n + s;
   d->primed = true;
   return 0;
+}
+
+int cthip_decoder_forward(void *dec, const float *tokens, int s, int n, int64_t *token, float *logits_out) {
+  CTHIP_REQUIRE_INIT();
+  CTHIP_ARG(dec != nullptr && tokens != nullptr && token != nullptr);
+  return forward_impl((Decoder *)dec, tokens, s, n, nullptr, 0, token, logits_out);
+}
+
+int cthip_decoder_forward_rows(void *dec, const float *tokens, int s, int n, const int *rows, int n_rows, int64_t *token,
+                               float *logits_out) {
+  CTHIP_REQUIRE_INIT();
+  CTHIP_ARG(dec != nullptr && tokens != nullptr && token != nullptr);
+  CTHIP_ARG(n_rows >= 0 && (n_rows == 0 || (rows != nullptr && logits_out != nullptr)));
+  for (int r = 0; r < n_rows; r++)
+    if (rows[r] < 0 || rows[r] >= s) return fail(CTHIP_E_BAD_ARG, "cthip_decoder_forward_rows: row %d of a forward of %d tokens", rows[r], s);
+  static const int none = 0;
+  return forward_impl((Decoder *)dec, tokens, s, n, n_rows ? rows : &none, n_rows, token, logits_out);
 }
 
 // the loop behind cthip_decoder_generate / cthip_decoder_generate_until
@@ -1222,6 +1277,7 @@ int cthip_decoder_layer_launches(void *dec) {
   Decoder *d = (Decoder *)dec;
   int rc = finalize(d);
   if (rc) return -1;
+  if (d->cfg.arch == CTHIP_ARCH_MIXED) return mixed_launches(d);
   if (d->flow) return 1;  // all layers are ONE launch
   if (d->fused || d->fused_gqa) return 3;  // (GPT-2 shapes: also over a cache of Q8_0 rows)
   return 5;  // (Q8_0 and paged caches too: rotation, quantisation / copy and append of the new row happen inside the attention launch)
@@ -1232,7 +1288,8 @@ int64_t cthip_decoder_step_bytes(const void *dec, int t) {
   if (!d || !d->finalized) return -1;
   const cthip_decoder_config &c = d->cfg;
   const int64_t KD = kv_dim(c);
-  int64_t emb = 4LL * c.dim * (c.arch == CTHIP_ARCH_GPT2 ? 2 : 1);
+  int64_t emb = 4LL * c.dim * (d->wpe ? 2 : 1);
+  if (c.arch == CTHIP_ARCH_MIXED) return d->weight_bytes + d->vector_bytes + emb + mixed_state_bytes(d, t);
   // per element of a cache row: 4 bytes, or 1 + 2 / 32 as Q8_0
   int64_t kv_read = d->kvq ? 2LL * c.n_layers * t * (KD + KD / 32 * 2) : 2LL * c.n_layers * t * KD * 4;
   int64_t kv_write = d->kvq ? 2LL * c.n_layers * (KD + KD / 32 * 2) : 2LL * c.n_layers * KD * 4;
@@ -1249,6 +1306,7 @@ int cthip_decoder_peek(void *dec, const char *what, void **ptr, int64_t *n_float
   int64_t n = 0;
   void *p = nullptr;
   int l = -1;
+  if (c.arch == CTHIP_ARCH_MIXED && (rc = mixed_peek(d, what, ptr, n_floats)) <= 0) return rc;
   if (!strcmp(what, "logits")) {
     p = d->logits;
     n = c.vocab;
@@ -1259,7 +1317,7 @@ int cthip_decoder_peek(void *dec, const char *what, void **ptr, int64_t *n_float
     // int64 clock stamps [workgroups][n_layers][4]; n counts their bytes in units of four
     p = d->flow_args.trace;
     n = (int64_t)dec_flow_grid(c.dim, c.n_heads, c.ffn) * c.n_layers * 4 * 2;
-  } else if ((sscanf(what, "k_cache.%d", &l) == 1 || sscanf(what, "v_cache.%d", &l) == 1) && l >= 0 && l < c.n_layers) {
+  } else if ((sscanf(what, "k_cache.%d", &l) == 1 || sscanf(what, "v_cache.%d", &l) == 1) && l >= 0 && l < (int)d->layers.size()) {
     const bool key = what[0] == 'k';
     n = (int64_t)c.max_seq * kv_dim(c);
     if (d->kvp) {

@@ -26,6 +26,10 @@ template <>
 struct Fmt<CTHIP_F16> {
   static constexpr int XPC = 8;
 };
+template <>
+struct Fmt<CTHIP_BF16> {
+  static constexpr int XPC = 8;
+};
 
 template <int TYPE>
 __device__ __forceinline__ float chunk_dot(const uint4 w, float scale, const float *__restrict__ x, float xsum);
@@ -87,6 +91,18 @@ __device__ __forceinline__ float chunk_dot<CTHIP_F16>(const uint4 w, float, cons
   return s;
 }
 
+template <>
+__device__ __forceinline__ float chunk_dot<CTHIP_BF16>(const uint4 w, float, const float *__restrict__ x, float) {
+  const uint32_t dw[4] = {w.x, w.y, w.z, w.w};
+  float s = 0.0f;
+#pragma unroll
+  for (int t = 0; t < 4; t++) {  // a bf16 is the upper half of the float it stands for
+    s = fmaf(__uint_as_float(dw[t] << 16), x[2 * t], s);
+    s = fmaf(__uint_as_float(dw[t] & 0xffff0000u), x[2 * t + 1], s);
+  }
+  return s;
+}
+
 // lowest-index argmax merge: (v, i) <- better of (v, i) and (ov, oi)
 __device__ __forceinline__ void argmax_merge(float &v, int &i, float ov, int oi) {
   if (ov > v || (ov == v && oi < i)) {
@@ -100,6 +116,7 @@ __device__ __forceinline__ float gemv_store(const GemvArgs &a, int m, int row, f
                                             float resid) {
   float v = acc + bias;
   v = apply_act(a.act, v);
+  if (a.softcap > 0.0f) v = softcap(v, a.softcap);
   v += resid;
   float *dst;
   if (row < a.split1) {
@@ -808,8 +825,8 @@ constexpr gemv_fn gemv_pair_fn() {
    {k_gemv<T, G, KC, PD_OF_T(T, KC), false, false, PD_OF_T(T, KC) != 1>, k_gemv<T, G, KC, PD_OF_T(T, KC), true, false, PD_OF_T(T, KC) != 1>}, \
    {k_gemv<T, G, KC, 1, false>, k_gemv<T, G, KC, 1, true>},                                              \
    {gemv_pair_fn<T, G, KC, false>(), gemv_pair_fn<T, G, KC, true>()}},
-// defined in gemv_q8.hip, gemv_q4.hip, gemv_f32.hip, gemv_f16.hip
-extern const GemvVariant kGemvQ8[], kGemvQ4[], kGemvF32[], kGemvF16[];
-extern const int kGemvQ8Count, kGemvQ4Count, kGemvF32Count, kGemvF16Count;
+// defined in gemv_q8.hip, gemv_q4.hip, gemv_f32.hip, gemv_f16.hip, gemv_bf16.hip
+extern const GemvVariant kGemvQ8[], kGemvQ4[], kGemvF32[], kGemvF16[], kGemvBF16[];
+extern const int kGemvQ8Count, kGemvQ4Count, kGemvF32Count, kGemvF16Count, kGemvBF16Count;
 
 }  // namespace cthip

@@ -20,6 +20,10 @@ namespace cthip {
 #define GEMV_SHAPES_F16(V) V(CTHIP_F16, 16, 2) V(CTHIP_F16, 64, 1) V(CTHIP_F16, 64, 2) V(CTHIP_F16, 64, 3) V(CTHIP_F16, 64, 4) \
   V(CTHIP_F16, 64, 6) V(CTHIP_F16, 64, 8) V(CTHIP_F16, 64, 12)
 
+// (bf16 chunks hold as many weights as fp16 ones: the same shapes)
+#define GEMV_SHAPES_BF16(V) V(CTHIP_BF16, 16, 2) V(CTHIP_BF16, 64, 1) V(CTHIP_BF16, 64, 2) V(CTHIP_BF16, 64, 3) V(CTHIP_BF16, 64, 4) \
+  V(CTHIP_BF16, 64, 6) V(CTHIP_BF16, 64, 8) V(CTHIP_BF16, 64, 12)
+
 // looping launches keep about 12 sixteen-byte loads per lane in flight; the widest 4-bit variants (96+ input floats per
 // lane in registers) keep two tiles, which leaves room for a second wavefront per SIMD
 #define PD_OF_T(T, KC) (KC >= 12 ? 1 : (KC >= 6 || ((T) == CTHIP_Q4_0 && KC >= 3)) ? 2 : 4)
@@ -33,6 +37,7 @@ inline const std::vector<GemvShape> &gemv_shapes() {
   static const std::vector<GemvShape> all = {
 #define GEMV_SHAPE_ENTRY(T, G, KC) {T, G, KC},
       GEMV_SHAPES_Q8(GEMV_SHAPE_ENTRY) GEMV_SHAPES_Q4(GEMV_SHAPE_ENTRY) GEMV_SHAPES_F32(GEMV_SHAPE_ENTRY) GEMV_SHAPES_F16(GEMV_SHAPE_ENTRY)
+      GEMV_SHAPES_BF16(GEMV_SHAPE_ENTRY)
 #undef GEMV_SHAPE_ENTRY
   };
   return all;
@@ -42,7 +47,7 @@ inline int gemv_xpc(int type) {  // input elements one 16-byte chunk multiplies
   switch (type) {
     case CTHIP_Q8_0: return 16;
     case CTHIP_Q4_0: return 32;
-    case CTHIP_F16: return 8;
+    case CTHIP_F16: case CTHIP_BF16: return 8;
     default: return 4;
   }
 }
@@ -198,7 +203,7 @@ struct GemvWidePlan {
 constexpr size_t kGemvWideMaxLdsBytes = 150 * 1024;
 inline GemvWidePlan gemv_wide_plan(int type, long long rows, long long cols, int compute_units) {
   GemvWidePlan p;
-  if (type != CTHIP_Q8_0 && type != CTHIP_Q4_0 && type != CTHIP_F16 && type != CTHIP_F32) return p;
+  if (type != CTHIP_Q8_0 && type != CTHIP_Q4_0 && type != CTHIP_F16 && type != CTHIP_BF16 && type != CTHIP_F32) return p;
   const int xpc = gemv_xpc(type);
   const bool quant = type == CTHIP_Q8_0 || type == CTHIP_Q4_0;
   if (rows <= 0 || rows > 0x7fffffff || cols < 64 || cols % (quant ? 32 : xpc) || cols > 0x7fffffff) return p;

@@ -222,6 +222,7 @@ int launch_gemv_wide(const WMat *w, GemvArgs a, int m) {
   PICK(CTHIP_Q4_0, 1)
   PICK(CTHIP_Q8_0, 1) PICK(CTHIP_Q8_0, 2) PICK(CTHIP_Q8_0, 3)
   PICK(CTHIP_F16, 1) PICK(CTHIP_F16, 2) PICK(CTHIP_F16, 3)
+  PICK(CTHIP_BF16, 1) PICK(CTHIP_BF16, 2) PICK(CTHIP_BF16, 3)
   PICK(CTHIP_F32, 1) PICK(CTHIP_F32, 2) PICK(CTHIP_F32, 3)
 #undef PICK
   // 8-bit rows, one per wavefront and tile, no wavefront with more than six (eight) tiles: a ring of six (eight), so

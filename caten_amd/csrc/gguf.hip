@@ -115,7 +115,7 @@ static bool skip_value(Cursor &c, uint32_t type, GGUFValue *out) {
 static uint64_t tensor_nbytes(uint32_t type, uint64_t n) {
   switch (type) {
     case CTHIP_F32: return n * 4;
-    case CTHIP_F16: return n * 2;
+    case CTHIP_F16: case CTHIP_BF16: return n * 2;
     case CTHIP_Q8_0: return (n + 31) / 32 * 34;
     case CTHIP_Q4_0: return n / 32 * 18;
     default: return 0;  // other ggml types: known ids (tensor-info.lisp:3-31), no decoder here either
@@ -363,7 +363,7 @@ int cthip_decoder_load_gguf(void *dec, const void *h, int arch, int *n_loaded) {
     const GGUFTensor &t = g->tensors[i];
     const std::string key = arch == CTHIP_ARCH_GPT2 ? remap_gpt2(t.name) : remap_llama(t.name);
     if (t.nbytes == 0)
-      return fail(CTHIP_E_UNSUPPORTED, "cthip_decoder_load_gguf: tensor '%s' has ggml type %u (supported: F32, F16, Q4_0, Q8_0)",
+      return fail(CTHIP_E_UNSUPPORTED, "cthip_decoder_load_gguf: tensor '%s' has ggml type %u (supported: F32, F16, BF16, Q4_0, Q8_0)",
                   t.name.c_str(), t.type);
     // dims are stored innermost first; (rows, cols) = (product of the outer dims, dims[0]) (tensor-info.lisp:104-120)
     int64_t rows = 1;

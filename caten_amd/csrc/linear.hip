@@ -5,7 +5,7 @@
 //
 // HBM layout of a packed matrix (rows x cols):
 //   quant plane  Q8_0: int8  [rows][cols]      Q4_0: u8 [rows][cols/2]
-//                F32 : float [rows][cols]      F16 : half [rows][cols]
+//                F32 : float [rows][cols]      F16, BF16 : 16-bit floats [rows][cols]
 //   scale plane  fp16 [rows][cols/32]          (quantised types only)
 // Q4_0 keeps ggml's nibble order inside each 16-byte block (low nibbles are
 // elements 0..15, high nibbles 16..31).  Total bytes equal the GGUF bytes, but
@@ -68,6 +68,12 @@ __global__ void k_dequant_f32_raw(const uint8_t *__restrict__ raw, int64_t n, fl
   out[i] = __uint_as_float(u);
 }
 
+__global__ void k_dequant_bf16_raw(const uint8_t *__restrict__ raw, int64_t n, float *__restrict__ out) {
+  int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= n) return;
+  out[i] = bf16_bits_to_float((unsigned short)(raw[2 * i] | (raw[2 * i + 1] << 8)));
+}
+
 // GGUF blocks -> planes. One thread per block.
 __global__ void k_repack_q8_0(const uint8_t *__restrict__ raw, int64_t nblocks, uint32_t *__restrict__ q,
                               unsigned short *__restrict__ d) {
@@ -110,6 +116,8 @@ __global__ void k_wmat_dequant(int type, const void *__restrict__ qp, const unsi
     out[i] = (float)(nib - 8) * half_bits_to_float(dp[b]);
   } else if (type == CTHIP_F16) {
     out[i] = half_bits_to_float(((const unsigned short *)qp)[i]);
+  } else if (type == CTHIP_BF16) {
+    out[i] = bf16_bits_to_float(((const unsigned short *)qp)[i]);
   } else {
     out[i] = ((const float *)qp)[i];
   }
@@ -258,7 +266,9 @@ __global__ __launch_bounds__(256) void k_gemv_elements(GemvArgs a) {
     float acc = 0.0f;
     for (int c = lane; c < a.cols; c += 64) {
       const int64_t e = (int64_t)row * a.cols + c;
-      const float w = TYPE == CTHIP_F16 ? half_bits_to_float(((const unsigned short *)a.q)[e]) : ((const float *)a.q)[e];
+      const float w = TYPE == CTHIP_F16    ? half_bits_to_float(((const unsigned short *)a.q)[e])
+                      : TYPE == CTHIP_BF16 ? bf16_bits_to_float(((const unsigned short *)a.q)[e])
+                                           : ((const float *)a.q)[e];
       acc = fmaf(w, x[c], acc);
     }
     acc = wave_sum(acc);
@@ -319,6 +329,7 @@ static const std::vector<GemvVariant> &all_variants() {
     v.insert(v.end(), kGemvQ4, kGemvQ4 + kGemvQ4Count);
     v.insert(v.end(), kGemvF32, kGemvF32 + kGemvF32Count);
     v.insert(v.end(), kGemvF16, kGemvF16 + kGemvF16Count);
+    v.insert(v.end(), kGemvBF16, kGemvBF16 + kGemvBF16Count);
     return v;
   }();
   return all;
@@ -544,6 +555,10 @@ int launch_gemv(const WMat *w, GemvArgs a, int m) {
       if (chunks) hipLaunchKernelGGL(k_gemv_generic<CTHIP_F16>, grid, block, 0, s.stream, a);
       else hipLaunchKernelGGL(k_gemv_elements<CTHIP_F16>, grid, block, 0, s.stream, a);
       break;
+    case CTHIP_BF16:
+      if (chunks) hipLaunchKernelGGL(k_gemv_generic<CTHIP_BF16>, grid, block, 0, s.stream, a);
+      else hipLaunchKernelGGL(k_gemv_elements<CTHIP_BF16>, grid, block, 0, s.stream, a);
+      break;
     default:
       if (chunks) hipLaunchKernelGGL(k_gemv_generic<CTHIP_F32>, grid, block, 0, s.stream, a);
       else hipLaunchKernelGGL(k_gemv_elements<CTHIP_F32>, grid, block, 0, s.stream, a);
@@ -619,6 +634,7 @@ int cthip_dequant(int ggml_type, const void *raw, int64_t n, float *out) {
       hipLaunchKernelGGL(k_dequant_q4_0_raw, grid, block, 0, st, (const uint8_t *)raw, n, out);
       break;
     case CTHIP_F16: hipLaunchKernelGGL(k_dequant_f16_raw, grid, block, 0, st, (const uint8_t *)raw, n, out); break;
+    case CTHIP_BF16: hipLaunchKernelGGL(k_dequant_bf16_raw, grid, block, 0, st, (const uint8_t *)raw, n, out); break;
     case CTHIP_F32: hipLaunchKernelGGL(k_dequant_f32_raw, grid, block, 0, st, (const uint8_t *)raw, n, out); break;
     default:
       // tensor-info.lisp:36-41 signals "Not ready" for every other ggml type
@@ -631,7 +647,7 @@ int cthip_dequant(int ggml_type, const void *raw, int64_t n, float *out) {
 int cthip_wmat_create(void **wmat, int ggml_type, const void *raw, int64_t rows, int64_t cols) {
   CTHIP_REQUIRE_INIT();
   CTHIP_ARG(wmat != nullptr && raw != nullptr && rows > 0 && cols > 0);
-  if (ggml_type != CTHIP_Q8_0 && ggml_type != CTHIP_Q4_0 && ggml_type != CTHIP_F32 && ggml_type != CTHIP_F16)
+  if (ggml_type != CTHIP_Q8_0 && ggml_type != CTHIP_Q4_0 && ggml_type != CTHIP_F32 && ggml_type != CTHIP_F16 && ggml_type != CTHIP_BF16)
     return fail(CTHIP_E_UNSUPPORTED, "cthip_wmat_create: ggml type %d is not supported", ggml_type);
   if ((ggml_type == CTHIP_Q8_0 || ggml_type == CTHIP_Q4_0) && cols % 32)
     return fail(CTHIP_E_BAD_ARG, "cthip_wmat_create: quantised rows need cols %% 32 == 0, got %lld", (long long)cols);

@@ -59,7 +59,7 @@ struct GemmArgs {
 // holds them k-contiguous per row in bf16, 16-byte chunks swizzled by row so that neither the operand
 // reads nor the staging writes collide on banks.  Two LDS buffers and three register sets keep the
 // global loads three K-steps ahead of the MFMAs with one barrier per step.
-enum { W_ROWMAJOR = 0, W_F32 = 1, W_F16 = 2, W_Q4 = 3, W_Q8 = 4 };  // W_Q4 / W_Q8: k_gemm_qpc only
+enum { W_ROWMAJOR = 0, W_F32 = 1, W_F16 = 2, W_Q4 = 3, W_Q8 = 4, W_BF16 = 5 };  // W_Q4 / W_Q8: k_gemm_qpc only
 typedef __bf16 v8bf __attribute__((ext_vector_type(8)));
 typedef __bf16 v2bf __attribute__((ext_vector_type(2)));
 typedef float v2f __attribute__((ext_vector_type(2)));
@@ -112,7 +112,7 @@ struct ARegs {  // one K-step of A held by a thread: rows ar + 16 i
 typedef unsigned v4u __attribute__((ext_vector_type(4)));
 template <int BMODE>
 struct BRegs {  // one K-step of B held by a thread between its request and its conversion
-  static constexpr int NV = (BMODE == W_ROWMAJOR || BMODE == W_F32) ? 4 : (BMODE == W_F16 ? 2 : 1);
+  static constexpr int NV = (BMODE == W_ROWMAJOR || BMODE == W_F32) ? 4 : (BMODE == W_F16 || BMODE == W_BF16 ? 2 : 1);
   v4u v[NV];
 };
 
@@ -185,6 +185,7 @@ __device__ __forceinline__ void store_tile(const GemmArgs &a, const float *Cs, i
 template <int BMODE, int NS, bool AL>
 __global__ __launch_bounds__(768) void k_gemm_split(GemmArgs a) {
   constexpr int BM = 64, BN = 64, BK = 64, LDK = BK, NP = (NS == 1) ? 1 : (NS == 3) ? 2 : 3;
+  constexpr int NPB = BMODE == W_BF16 ? 1 : NP;  // a bf16 weight is its own leading term, the others are zero
   constexpr int NSET = 3;  // register sets = K-steps of global loads in flight
   constexpr int kOpBytes = 2 * NP * BM * LDK * 2, kCBytes = BM * (BN + 4) * 4;
   // both operand buffers; after the last step the same memory holds the output tile (store_tile)
@@ -254,7 +255,7 @@ __global__ __launch_bounds__(768) void k_gemm_split(GemmArgs a) {
         rb.v[BRegs<BMODE>::NV > 1 ? 1 : 0] = src[st];
         rb.v[BRegs<BMODE>::NV > 2 ? 2 : 0] = src[2 * st];
         rb.v[BRegs<BMODE>::NV > 3 ? 3 : 0] = src[3 * st];
-      } else if (BMODE == W_F16) {
+      } else if (BMODE == W_F16 || BMODE == W_BF16) {
         const v4u *src = ok ? (const v4u *)((const unsigned short *)a.wq + e) : (const v4u *)g_zeros;
         rb.v[0] = src[0];
         rb.v[BRegs<BMODE>::NV > 1 ? 1 : 0] = src[1];
@@ -289,6 +290,10 @@ __global__ __launch_bounds__(768) void k_gemm_split(GemmArgs a) {
       put(1, q0.y, q1.y, q2.y, q3.y);
       put(2, q0.z, q1.z, q2.z, q3.z);
       put(3, q0.w, q1.w, q2.w, q3.w);
+    } else if (BMODE == W_BF16) {  // the bytes as they are
+#pragma unroll
+      for (int j = 0; j < 2; j++)
+        *(v4u *)&Bs[buf][0][wr][8 * ((2 * wkc + j) ^ swz(wr))] = rb.v[BRegs<BMODE>::NV > 1 ? j : 0];
     } else {
       float x[16];
       if (BMODE == W_F32) {
@@ -328,14 +333,14 @@ __global__ __launch_bounds__(768) void k_gemm_split(GemmArgs a) {
   auto mma = [&](int buf) __attribute__((always_inline)) {
     // 32x32x16: lane l holds A[i = l%32][k = 8*(l/32) .. +7] and B[k = 8*(l/32) .. +7][j = l%32]
     const int rowa = 32 * wm + (lane & 31), rowb = 32 * wn + (lane & 31);
-    v8bf av[BK / 16][NP], bv[BK / 16][NP];
+    v8bf av[BK / 16][NP], bv[BK / 16][NPB];
 #pragma unroll
     for (int s = 0; s < BK / 16; s++) {
       const int ch = 2 * s + (lane >> 5);
 #pragma unroll
       for (int p = 0; p < NP; p++) {
         av[s][p] = __builtin_bit_cast(v8bf, *(const uint4 *)&As[buf][p][rowa][8 * (ch ^ swz(rowa))]);
-        bv[s][p] = __builtin_bit_cast(v8bf, *(const uint4 *)&Bs[buf][p][rowb][8 * (ch ^ swz(rowb))]);
+        if (p < NPB) bv[s][p] = __builtin_bit_cast(v8bf, *(const uint4 *)&Bs[buf][p][rowb][8 * (ch ^ swz(rowb))]);
       }
     }
     __builtin_amdgcn_sched_barrier(0);
@@ -345,7 +350,8 @@ __global__ __launch_bounds__(768) void k_gemm_split(GemmArgs a) {
 #pragma unroll
       for (int t = NP - 1; t >= 0; t--) {
 #pragma unroll
-        for (int p = 0; p <= t; p++) acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(av[s][p], bv[s][t - p], acc, 0, 0, 0);
+        for (int p = 0; p <= t; p++)
+          if (t - p < NPB) acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(av[s][p], bv[s][t - p], acc, 0, 0, 0);
       }
     }
   };
@@ -684,7 +690,7 @@ __global__ __launch_bounds__(256 + 64 * NPW) void k_gemm_qpc(GemmArgs a) {
 
 // ---------------------------------------------------------------------------------------------
 // fp32-operand MFMA GEMM (v_mfma_f32_32x32x2_f32): the products are fp32 products, only the summation
-// order differs from a scalar loop.  This kernel takes PACKED WEIGHTS (N rows x K, any of the five formats,
+// order differs from a scalar loop.  This kernel takes PACKED WEIGHTS (N rows x K, any of the formats,
 // dequantised to fp32 while staging); a (K,N) fp32 matrix takes k_gemm_f32pc below.  64x64 tile per 256-thread
 // workgroup, 2x2 wavefronts, two LDS buffers, three register sets of global loads in flight, one barrier per
 // step, XCD regions, split-K, K-steps of 32, the operands kept as fp32 in LDS, k-major ([k][m], [k][n]):
@@ -758,7 +764,7 @@ __global__ __launch_bounds__(256) void k_gemm_f32(GemmArgs a) {
         const uint4 *src = in ? (const uint4 *)((const float *)a.wq + e) : (const uint4 *)z;
         rb.r0 = src[0];
         rb.r1 = src[1];
-      } else if (a.wtype == CTHIP_F16) {
+      } else if (a.wtype == CTHIP_F16 || a.wtype == CTHIP_BF16) {
         rb.r0 = *(in ? (const uint4 *)((const unsigned short *)a.wq + e) : (const uint4 *)z);
       } else {
         // Q8_0: 8 int8.  Q4_0: elements j < 16 of a block are the low nibbles of its bytes j, j >= 16 the high
@@ -791,6 +797,11 @@ __global__ __launch_bounds__(256) void k_gemm_f32(GemmArgs a) {
         w2 = half_bits_to_float((unsigned short)(rb.r0.y & 0xffff)), w3 = half_bits_to_float((unsigned short)(rb.r0.y >> 16));
         w4 = half_bits_to_float((unsigned short)(rb.r0.z & 0xffff)), w5 = half_bits_to_float((unsigned short)(rb.r0.z >> 16));
         w6 = half_bits_to_float((unsigned short)(rb.r0.w & 0xffff)), w7 = half_bits_to_float((unsigned short)(rb.r0.w >> 16));
+      } else if (a.wtype == CTHIP_BF16) {
+        w0 = __uint_as_float(rb.r0.x << 16), w1 = __uint_as_float(rb.r0.x & 0xffff0000u);
+        w2 = __uint_as_float(rb.r0.y << 16), w3 = __uint_as_float(rb.r0.y & 0xffff0000u);
+        w4 = __uint_as_float(rb.r0.z << 16), w5 = __uint_as_float(rb.r0.z & 0xffff0000u);
+        w6 = __uint_as_float(rb.r0.w << 16), w7 = __uint_as_float(rb.r0.w & 0xffff0000u);
       } else if (a.wtype == CTHIP_Q8_0) {
         const float d = half_bits_to_float(rb.d);
         const int v0 = (int)rb.r0.x, v1 = (int)rb.r0.y;
@@ -1137,7 +1148,7 @@ int launch_gemm(GemmArgs a, int bmode, int precision, float *static_ws, size_t s
     // one region of tiles per XCD: the split with the fewest tiles per XCD, then the least operand bytes per L2
     a.tm = (a.M + bm - 1) / bm;
     a.tn = (a.N + bn - 1) / bn;
-    const double sza = 4.0 * bm / 64, szb = bmode == B_ROWMAJOR ? 4.0 : a.wtype == CTHIP_Q8_0 ? 1.0625 : a.wtype == CTHIP_Q4_0 ? 0.5625 : a.wtype == CTHIP_F16 ? 2.0 : 4.0;
+    const double sza = 4.0 * bm / 64, szb = bmode == B_ROWMAJOR ? 4.0 : a.wtype == CTHIP_Q8_0 ? 1.0625 : a.wtype == CTHIP_Q4_0 ? 0.5625 : a.wtype == CTHIP_F16 || a.wtype == CTHIP_BF16 ? 2.0 : 4.0;
     double best = -1.0;
     for (int rx = 1; rx <= 8; rx *= 2) {
       const int ry = 8 / rx, rm = (a.tm + rx - 1) / rx, rn = (a.tn + ry - 1) / ry;
@@ -1215,7 +1226,7 @@ int launch_gemm(GemmArgs a, int bmode, int precision, float *static_ws, size_t s
 #undef QG
   } else {
     int wm = W_ROWMAJOR;
-    if (bmode == B_WMAT) wm = a.wtype == CTHIP_F16 ? W_F16 : W_F32;
+    if (bmode == B_WMAT) wm = a.wtype == CTHIP_F16 ? W_F16 : a.wtype == CTHIP_BF16 ? W_BF16 : W_F32;
 #define SPLIT3(MODE, AL)                                                                                      \
   if (precision == GEMM_BF16X6) hipLaunchKernelGGL((k_gemm_split<MODE, 6, AL>), grid, dim3(768), 0, st, a);      \
   else if (precision == GEMM_BF16X3) hipLaunchKernelGGL((k_gemm_split<MODE, 3, AL>), grid, dim3(768), 0, st, a); \
@@ -1234,6 +1245,7 @@ int launch_gemm(GemmArgs a, int bmode, int precision, float *static_ws, size_t s
       SPLIT(W_ROWMAJOR);
       SPLIT(W_F32);
       SPLIT(W_F16);
+      SPLIT(W_BF16);
     }
 #undef SPLIT3
 #undef SPLIT

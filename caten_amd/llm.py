@@ -9,12 +9,14 @@ device-resident decoder session of libcaten_hip.so.
 from __future__ import annotations
 
 import ctypes as C
+import json
+import os
 from typing import Dict, List, Optional, Sequence, Tuple
 
 import numpy as np
 
-from . import _lib
-from .quant import quantize, packed_nbytes
+from . import _lib, safetensors
+from .quant import from_bf16, packed_nbytes, quantize, to_bf16
 
 # *remap-key* (apps/gpt2/gpt2.lisp:52-70): GGUF tensor names -> Caten state-dict keys
 GPT2_REMAP = [
@@ -53,6 +55,8 @@ class Tensor:
             return cls(kind, a.view(np.uint8), rows, cols)
         if kind == "f16":
             return cls(kind, a.astype(np.float16).view(np.uint8), rows, cols)
+        if kind == "bf16":
+            return cls(kind, to_bf16(a).view(np.uint8), rows, cols)
         return cls(kind, quantize(kind, a), rows, cols)
 
 
@@ -97,6 +101,11 @@ class Transformer:
         self.cfg = dict(cfg)
         self.arch = arch
         self.lib = _lib.init(device)
+        self.handle = C.c_void_p()
+        self._create(cfg)
+
+    def _create(self, cfg: dict) -> None:
+        arch = self.arch
         c = _lib.DecoderConfig()
         c.arch = _lib.ARCH_GPT2 if arch == "gpt2" else _lib.ARCH_LLAMA
         c.n_layers, c.dim, c.n_heads = cfg["n_layers"], cfg["dim"], cfg["n_heads"]
@@ -104,7 +113,6 @@ class Transformer:
         c.ffn, c.vocab, c.max_seq = cfg["ffn"], cfg["vocab"], cfg["max_seq"]
         c.eps = cfg.get("eps", 1e-5)
         c.rope_base = cfg.get("rope_base", 10000.0)
-        self.handle = C.c_void_p()
         _lib.check(self.lib.cthip_decoder_create(C.byref(self.handle), C.byref(c)))
 
     def load_state_dict(self, sd: Dict[str, Tensor]) -> "Transformer":
@@ -128,6 +136,17 @@ class Transformer:
         _lib.check(self.lib.cthip_decoder_forward(self.handle, toks.ctypes.data, s, n, C.byref(tok),
                                                   logits.ctypes.data if return_logits else None))
         return (int(tok.value), logits) if return_logits else int(tok.value)
+
+    def forward_rows(self, x: Sequence[float], rows: Sequence[int], n: int = 0) -> Tuple[int, np.ndarray]:
+        """forward, with the logits of the listed positions of x: (greedy token of the last one, (len(rows), vocab))"""
+        toks = np.ascontiguousarray(x, np.float32).ravel()
+        idx = np.ascontiguousarray(rows, np.int32).ravel()
+        out = np.empty((idx.size, self.cfg["vocab"]), np.float32)
+        tok = C.c_int64()
+        _lib.check(self.lib.cthip_decoder_forward_rows(self.handle, toks.ctypes.data, toks.size, n,
+                                                       idx.ctypes.data_as(C.POINTER(C.c_int)), idx.size, C.byref(tok),
+                                                       out.ctypes.data))
+        return int(tok.value), out
 
     def generate_until(self, max_steps: int, eos_token: int) -> List[int]:
         """Greedy tokens from the device-resident loop until `eos_token` has been produced (it is the last element)
@@ -176,6 +195,86 @@ def make_gpt2(cfg: dict, state_dict: Dict[str, Tensor], device: int = 0) -> Tran
 
 def make_llama(cfg: dict, state_dict: Dict[str, Tensor], device: int = 0) -> Transformer:
     return Transformer(cfg, "llama", device).load_state_dict(state_dict)
+
+
+class MixedTransformer(Transformer):
+    """A decoder whose layers are listed one by one (cthip_decoder_create_mixed).  cfg: `vocab`, `dim`, `max_seq`, `eps`,
+    `norm` ("layernorm" or "rmsnorm"), `position_base`, `logit_softcap` (0 = none), `precision` (operand format of the
+    products over several rows, None = the library's option) and `layers`, each a dict of `mixer` ("delta" or
+    "latent"), that mixer's sizes and `ffn` (0 = none)."""
+
+    MIXERS = {"delta": _lib.MIXER_DELTA, "latent": _lib.MIXER_LATENT}
+    NORMS = {"layernorm": _lib.PRO_LAYERNORM, "rmsnorm": _lib.PRO_RMSNORM}
+
+    def __init__(self, cfg: dict, device: int = 0):
+        super().__init__(cfg, "mixed", device)
+
+    def _create(self, cfg: dict) -> None:
+        c = _lib.MixedConfig()
+        c.n_layers, c.dim, c.vocab, c.max_seq = len(cfg["layers"]), cfg["dim"], cfg["vocab"], cfg["max_seq"]
+        c.norm, c.eps = self.NORMS[cfg.get("norm", "layernorm")], cfg["eps"]
+        c.position_base, c.logit_softcap = cfg.get("position_base") or 0.0, cfg.get("logit_softcap") or 0.0
+        c.precision = -1 if cfg.get("precision") is None else cfg["precision"]
+        layers = (_lib.LayerSpec * len(cfg["layers"]))()
+        for s, l in zip(layers, cfg["layers"]):
+            s.mixer, s.heads, s.dim, s.vdim = self.MIXERS[l["mixer"]], l["heads"], l["dim"], l["vdim"]
+            s.kv_heads, s.conv = l.get("kv_heads", l["heads"]), l.get("conv", 0)
+            s.kv_rank, s.scale = l.get("kv_rank", 0), l.get("scale", 0.0)
+            s.sink, s.gate, s.ffn = int(l.get("sink", False)), int(l.get("gate", False)), l.get("ffn") or 0
+        _lib.check(self.lib.cthip_decoder_create_mixed(C.byref(self.handle), C.byref(c), layers))
+
+
+def zuselix_config(config: dict) -> dict:
+    """config.json of a Zuselix model -> MixedTransformer's cfg (without max_seq)"""
+    layers = []
+    for i, l in enumerate(config["layers"]):
+        m = dict(l["mixer"])
+        mlp = l.get("mlp")
+        if mlp is not None and mlp.get("kind", "dense") != "dense":
+            raise ValueError(f"layer {i}: a feed-forward of kind {mlp['kind']!r} is not part of this design")
+        m["ffn"] = int(mlp["ff"]) if mlp is not None else 0
+        if l["type"] == "delta":
+            m["mixer"] = "delta"
+        elif l["type"] == "latent_attention":
+            m.update(mixer="latent", sink=True, gate=True)
+        else:
+            raise ValueError(f"layer {i}: mixer type {l['type']!r} is not part of this design")
+        layers.append(m)
+    return dict(vocab=config["vocab"], dim=config["width"], eps=config["norm"]["eps"], norm="layernorm", position_base=10000.0,
+                logit_softcap=config.get("logit_softcap") or 0.0, layers=layers)
+
+
+# architecture name of a model directory's config.json -> (its configuration, the session's class)
+ARCHITECTURES = {"Zuselix": (zuselix_config, MixedTransformer)}
+
+
+def load_model(path: str, dtype: str = "bfloat16", max_seq: int = 2048, device: int = 0) -> Transformer:
+    """A model directory (config.json, model.safetensors) -> a session with its weights loaded.  dtype "bfloat16" keeps the
+    Linear weights in 16 bits as they are; "float32" widens them and multiplies fp32 operands everywhere."""
+    with open(os.path.join(path, "config.json")) as f:
+        config = json.load(f)
+    name = config.get("architecture")
+    if name not in ARCHITECTURES:
+        raise ValueError(f"{path}: architecture {name!r} is not registered (known: {', '.join(sorted(ARCHITECTURES))})")
+    if dtype not in ("bfloat16", "float32"):
+        raise ValueError(f"load_model: dtype {dtype!r} (bfloat16 or float32)")
+    to_cfg, cls = ARCHITECTURES[name]
+    cfg = dict(to_cfg(config), max_seq=max_seq)
+    if dtype == "float32":
+        cfg["precision"] = 0
+    tensors = safetensors.read(os.path.join(path, "model.safetensors"))
+    return cls(cfg, device).load_state_dict(safetensors_state_dict(tensors, widen=dtype == "float32"))
+
+
+def safetensors_state_dict(tensors: dict, widen: bool = False) -> Dict[str, Tensor]:
+    """tensors as safetensors.read gives them -> state dict; `widen`: bf16 values as fp32"""
+    sd = {}
+    for key, (kind, shape, raw) in tensors.items():
+        rows, cols = shape if len(shape) == 2 else (1, int(np.prod(shape)))
+        if widen and kind == "bf16":
+            kind, raw = "f32", from_bf16(np.ascontiguousarray(raw))
+        sd[key] = Tensor(kind, raw, rows, cols)
+    return sd
 
 
 def gpt2_generate(model: Transformer, prompt: Sequence[int], max_length: int = 100, on_device: bool = True,

@@ -13,7 +13,7 @@ import numpy as np
 BLOCK = 32
 BYTES_PER_BLOCK = {"q8_0": 34, "q4_0": 18}
 # ggml type ids (external/gguf/tensor-info.lisp:3-31)
-GGML_TYPE_ID = {"f32": 0, "f16": 1, "q4_0": 2, "q8_0": 8}
+GGML_TYPE_ID = {"f32": 0, "f16": 1, "q4_0": 2, "q8_0": 8, "bf16": 30}
 
 
 def _round_half_away(x):
@@ -48,6 +48,16 @@ def quantize_q4_0(w: np.ndarray) -> np.ndarray:
     return out.reshape(-1)
 
 
+def to_bf16(w: np.ndarray) -> np.ndarray:
+    """fp32 -> the bits of the nearest bf16 (ties to even)"""
+    u = np.ascontiguousarray(w, np.float32).view(np.uint32)
+    return ((u + np.uint32(0x7fff) + ((u >> np.uint32(16)) & np.uint32(1))) >> np.uint32(16)).astype(np.uint16)
+
+
+def from_bf16(bits: np.ndarray) -> np.ndarray:
+    return (np.asarray(bits).view(np.uint16).astype(np.uint32) << np.uint32(16)).view(np.float32)
+
+
 def quantize(kind: str, w: np.ndarray) -> np.ndarray:
     return {"q8_0": quantize_q8_0, "q4_0": quantize_q4_0}[kind](w)
 
@@ -55,6 +65,6 @@ def quantize(kind: str, w: np.ndarray) -> np.ndarray:
 def packed_nbytes(kind: str, n_elements: int) -> int:
     if kind == "f32":
         return 4 * n_elements
-    if kind == "f16":
+    if kind in ("f16", "bf16"):
         return 2 * n_elements
     return (n_elements + BLOCK - 1) // BLOCK * BYTES_PER_BLOCK[kind]

@@ -39,6 +39,7 @@ extern "C" {
 /* ggml tensor type ids (external/gguf/tensor-info.lisp:3-31) */
 #define CTHIP_F32 0
 #define CTHIP_F16 1
+#define CTHIP_BF16 30
 #define CTHIP_Q4_0 2
 #define CTHIP_Q8_0 8
 
@@ -355,6 +356,7 @@ int cthip_sdpa_cached_paged(float *out, const float *q, const void *const *k_pag
 
 #define CTHIP_ARCH_GPT2 0  /* LayerNorm, learned positions, fused qkv + biases, GELU MLP */
 #define CTHIP_ARCH_LLAMA 1 /* RMSNorm, RoPE, GQA, SwiGLU, no biases (not in the reference) */
+#define CTHIP_ARCH_MIXED 2 /* layers listed one by one (cthip_decoder_create_mixed; not in the reference) */
 
 typedef struct {
   int arch;
@@ -365,6 +367,41 @@ typedef struct {
 
 int cthip_decoder_create(void **dec, const cthip_decoder_config *cfg);
 int cthip_decoder_destroy(void *dec);
+
+/* A decoder whose layers are listed one by one, each with a token mixer and its sizes and, optionally, a SwiGLU
+ * feed-forward.  Pre-norm: x += mixer(norm1(x)), then x += ff(norm2(x)).  Such a session keeps, besides what a
+ * latent-attention layer caches, recurrent state that only moves forward: a forward starts at position 0 (a new
+ * sequence) or where the last one ended.  State-dict keys (i = layer; [rows, cols] as stored, y = W x):
+ *   embed [vocab, dim], final.norm, head [vocab, dim], l<i>.norm1, l<i>.norm2,
+ *   l<i>.mlp.gate / .up [ffn, dim], .down [dim, ffn]
+ *   CTHIP_MIXER_DELTA (gated delta rule): l<i>.mix.q / .k [kv_heads dim, width], .v [heads vdim, width], each with
+ *     .conv [channels, conv] (last column: the current token), .b / .a [heads, width], .A_log, .dt_bias [heads],
+ *     .g [heads vdim, width], .norm [vdim], .o [width, heads vdim]
+ *   CTHIP_MIXER_LATENT (attention over a cached latent): l<i>.mix.q [heads dim, width], .dkv [kv_rank, width],
+ *     .dkv.norm [kv_rank], .uk [heads dim, kv_rank], .uv [heads vdim, kv_rank], .o [width, heads vdim] and, where the
+ *     layer has them, .sink [heads] and .g [heads vdim, width]
+ * Linear weights are fp32, fp16 or bf16, one format per session. */
+#define CTHIP_MIXER_DELTA 0
+#define CTHIP_MIXER_LATENT 1
+typedef struct {
+  int mixer;           /* CTHIP_MIXER_* */
+  int heads, kv_heads; /* kv_heads: query / key heads of a delta layer, each shared by heads / kv_heads value heads */
+  int dim, vdim;       /* per head: query / key size, value size (at most 256) */
+  int conv;            /* delta: taps of the short convolutions */
+  int kv_rank;         /* latent: size of the cached vector (at most 1024) */
+  float scale;         /* latent: the scores' factor */
+  int sink, gate;      /* latent: 1 = the softmax has a sink / the output is gated */
+  int ffn;             /* feed-forward size, 0 = none */
+} cthip_layer_spec;
+typedef struct {
+  int n_layers, dim, vocab, max_seq;
+  int norm;            /* CTHIP_PRO_LAYERNORM (weight, no bias) or CTHIP_PRO_RMSNORM, everywhere */
+  float eps;
+  float position_base; /* > 0: a sinusoidal position vector of this base is added to the embedding */
+  float logit_softcap; /* > 0: logits = cap tanh(logits / cap) */
+  int precision;       /* operand format of the products over several rows, as option "gemm_precision"; -1 = that option */
+} cthip_mixed_config;
+int cthip_decoder_create_mixed(void **dec, const cthip_mixed_config *cfg, const cthip_layer_spec *layers);
 /* load-state-dict (source/api/module.lisp:290-320): hands one tensor to the
  * session under its reference state-dict key ("wte.weight", "h.3.attn.c_attn.weight",
  * "h.3.ln_1.affine", "ln_f.bias", "lm_head.weight", ... apps/gpt2/gpt2.lisp:52-70).
@@ -380,6 +417,10 @@ int cthip_decoder_missing(const void *dec);
  * to *token; logits_out (host, vocab floats) may be NULL.  Synchronous. */
 int cthip_decoder_forward(void *dec, const float *tokens, int s, int n, int64_t *token,
                           float *logits_out);
+/* The same, and the logits of `n_rows` of the s positions (rows[i] in 0 .. s-1) -> logits_out (host, n_rows x vocab
+ * floats): what scoring a prompt or replaying a trace needs. */
+int cthip_decoder_forward_rows(void *dec, const float *tokens, int s, int n, const int *rows, int n_rows, int64_t *token,
+                               float *logits_out);
 /* gpt2-generate's loop kept on the device: after a forward has left position
  * and last token on the device, runs `steps` further single-token forwards
  * without host round trips and writes their greedy tokens to tokens_out (host).
@@ -400,12 +441,15 @@ int64_t cthip_decoder_step_bytes(const void *dec, int t);
  * per-XCD accumulators -- taken only when the device passed the load-time checks that XCD ids are 0..7 and that
  * atomics of different workgroups of an XCD meet in its L2), 5 (one launch per Linear + attention; over Q8_0 cache
  * rows and over a paged cache the attention launch also rotates, quantises / copies and appends the new row).
- * A session of 3 runs 4 from position "attn_long_from" on.  -1 on error. */
+ * A session of 3 runs 4 from position "attn_long_from" on.  A mixed decoder: the most any of its layers runs.  -1 on
+ * error. */
 int cthip_decoder_layer_launches(void *dec);
 /* Device pointers into the session, for parity tests: "k_cache.<l>", "v_cache.<l>" (fp32 rows; with a Q8_0
  * cache their dequantised values, in a buffer the next peek overwrites), "logits", "x"; with a Q8_0 cache also
  * the planes themselves, "k_cache_q8.<l>" / "v_cache_q8.<l>" (int8[max_seq][kv_dim]) and "k_cache_d.<l>" /
- * "v_cache_d.<l>" (fp16[max_seq][kv_dim / 32]), n_floats counting their bytes in units of four. */
+ * "v_cache_d.<l>" (fp16[max_seq][kv_dim / 32]), n_floats counting their bytes in units of four.  A mixed decoder:
+ * "latent.<l>" (max_seq rows of the latent, padded to a multiple of 16), "state.<l>" ([head][value column][key], both
+ * padded likewise), "logits", "x". */
 int cthip_decoder_peek(void *dec, const char *what, void **ptr, int64_t *n_floats);
 
 /* ================================================================== */

@@ -67,7 +67,7 @@ static void walk(const Case &c) {
   const long long q0 = 16ll * (c.col0 / XPC), d0 = 2ll * (c.col0 >> 5), x0 = 4ll * c.col0, upo = full;
   const int in_cols = swiglu ? 2 * full : full;
   const long long x_stride = in_cols, out_rows = c.pair ? c.rows / 2 : c.rows, y_stride = out_rows;
-  const long long row_bytes = c.type == CTHIP_Q8_0 ? full : c.type == CTHIP_Q4_0 ? full / 2 : c.type == CTHIP_F16 ? 2ll * full : 4ll * full;
+  const long long row_bytes = c.type == CTHIP_Q8_0 ? full : c.type == CTHIP_Q4_0 ? full / 2 : c.type == CTHIP_F16 || c.type == CTHIP_BF16 ? 2ll * full : 4ll * full;
   Region Q = {"quant plane", true, row_bytes * c.rows}, D = {"scale plane", QUANT, 2ll * (full / 32) * c.rows};
   Region X = {"x", true, 4 * x_stride * c.m}, NG = {"norm_g", c.pro == CTHIP_PRO_LAYERNORM || c.pro == CTHIP_PRO_RMSNORM, 4ll * c.cols};
   Region NB = {"norm_b", layernorm, 4ll * c.cols}, B = {"bias", bias, 4ll * c.rows}, R = {"residual", c.residual, 4 * y_stride * c.m};
@@ -215,7 +215,7 @@ static void walk_wide(int type, int rows, int cols, int m_rows, int pro, bool bi
   const int nchunks = cols / XPC, n4 = cols >> 2, spr = cols >> 5;
   const long long x_stride = swiglu ? 2ll * cols : cols, y_stride = rows;
   const bool QUANT = Q4 || type == CTHIP_Q8_0;
-  const long long row_bytes = Q4 ? cols / 2 : type == CTHIP_Q8_0 ? cols : type == CTHIP_F16 ? 2ll * cols : 4ll * cols;
+  const long long row_bytes = Q4 ? cols / 2 : type == CTHIP_Q8_0 ? cols : type == CTHIP_F16 || type == CTHIP_BF16 ? 2ll * cols : 4ll * cols;
   Region Q = {"quant plane", true, row_bytes * rows}, D = {"scale plane", QUANT, 2ll * spr * rows};
   Region X = {"x", true, 4 * x_stride * m_rows}, NG = {"norm_g", rms && gamma, 4ll * cols}, B = {"bias", bias, 4ll * rows};
   Region R = {"residual", residual, 4 * y_stride * m_rows}, Y = {"y", true, 4 * y_stride * m_rows};
@@ -308,7 +308,7 @@ static void check_reduce_norm_plans() {
 }
 
 // "shape TYPE ROWS COLS [TYPE ROWS COLS ...]": only these Linears (TYPE = the library's code: 0 fp32, 1 fp16, 2 Q4_0,
-// 8 Q8_0), with every prologue and the flag sets a decoder launches -- for a model size outside the table below
+// 8 Q8_0, 30 bf16), with every prologue and the flag sets a decoder launches -- for a model size outside the table below
 static int walk_given_shapes(int argc, char **argv) {
   for (int i = 2; i + 2 < argc; i += 3) {
     const int type = atoi(argv[i]), rows = atoi(argv[i + 1]), cols = atoi(argv[i + 2]);
@@ -370,7 +370,7 @@ int main(int argc, char **argv) {
   check_reduce_norm_plans();
   // default: a few seconds (every shape, the flag combinations thinned out on the large ones); "full": everything
   const bool full = argc > 1 && !strcmp(argv[1], "full");
-  const int types[] = {CTHIP_Q8_0, CTHIP_Q4_0, CTHIP_F32, CTHIP_F16};
+  const int types[] = {CTHIP_Q8_0, CTHIP_Q4_0, CTHIP_F32, CTHIP_F16, CTHIP_BF16};
   // widths: each variant's exact width, one chunk less, the smallest, and the model widths
   const int rowsv[] = {1, 2, 3, 5, 17, 64, 767, 768, 2304, 3072, 5003, 32000, 50257};
   for (int type : types) {
@@ -420,7 +420,7 @@ int main(int argc, char **argv) {
     }
   }
   // the wide-row kernel on widths around its tile sizes, and rows fewer / more than wavefronts
-  for (int type : {CTHIP_Q8_0, CTHIP_Q4_0, CTHIP_F16, CTHIP_F32})
+  for (int type : {CTHIP_Q8_0, CTHIP_Q4_0, CTHIP_F16, CTHIP_BF16, CTHIP_F32})
     for (int cols : {64, 96, 2048, 2080, 4096, 5504, 6144, 8192, 8224, 11008})
       for (int rows : {1, 7, 513, 4100})
         for (int pro : {(int)CTHIP_PRO_NONE, (int)CTHIP_PRO_SWIGLU, (int)CTHIP_PRO_RMSNORM})
