@@ -383,7 +383,13 @@ def main():
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="also run one 256 MiB device-to-device copy (a kernel of known traffic to scale "
                          "rocprofv3 FETCH_SIZE / WRITE_SIZE readings by)")
+    ap.add_argument("--mixed", nargs="*", metavar="SIZE", default=None,
+                    help="instead of the headline workload: Zuselix shapes beside Llama shapes of equal size (bench_mixed.py)")
     args = ap.parse_args()
+    if args.mixed is not None:
+        import bench_mixed
+        bench_mixed.main(args.mixed)
+        return
     if args.gpus != 1:
         print("bench.py: this build measures one GPU only (batch-1 decode does not use a second); run with --gpus 1",
               file=sys.stderr)

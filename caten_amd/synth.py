@@ -97,6 +97,62 @@ def llama_weights(cfg: dict, seed: int = 0, threads: int = 1) -> dict:
     return w
 
 
+def _zuselix(width, ff, heads, kv_heads, rank, blocks, vocab=32000):
+    """blocks of two delta layers and a latent-attention layer, each with a feed-forward; heads of 128"""
+    delta = {"type": "delta", "mixer": dict(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, conv=4), "mlp": {"kind": "dense", "ff": ff}}
+    latent = {"type": "latent_attention", "mixer": dict(heads=heads, dim=128, vdim=128, kv_rank=rank, scale=128 ** -0.5),
+              "mlp": {"kind": "dense", "ff": ff}}
+    return {"architecture": "Zuselix", "layers": [delta, delta, latent] * blocks, "logit_softcap": 30.0, "norm": {"eps": 1e-5},
+            "vocab": vocab, "width": width}
+
+
+# config.json-shaped configurations beside Llama shapes of the same width, feed-forward, depth and vocabulary
+ZUSELIX_CONFIGS = {
+    "zuselix-1b": _zuselix(2048, 5632, 16, 8, 512, 7),
+    "zuselix-7b": _zuselix(4096, 11008, 32, 16, 512, 5),  # (15 of a 7B model's 32 layers)
+}
+
+
+def zuselix_shapes(config: dict) -> dict:
+    """tensor name -> shape of a Zuselix model (cthip_decoder_create_mixed's state-dict keys)"""
+    W, V = config["width"], config["vocab"]
+    out = {"embed": (V, W), "final.norm": (W,), "head": (V, W)}
+    for i, layer in enumerate(config["layers"]):
+        m, p = layer["mixer"], f"l{i}."
+        H, dk, dv = m["heads"], m["dim"], m["vdim"]
+        out.update({p + "norm1": (W,), p + "mix.q": (m.get("kv_heads", H) * dk, W), p + "mix.g": (H * dv, W), p + "mix.o": (W, H * dv)})
+        if layer["type"] == "delta":
+            K, taps = m["kv_heads"] * dk, m["conv"]
+            out.update({p + "mix.k": (K, W), p + "mix.v": (H * dv, W), p + "mix.q.conv": (K, taps), p + "mix.k.conv": (K, taps),
+                        p + "mix.v.conv": (H * dv, taps), p + "mix.b": (H, W), p + "mix.a": (H, W), p + "mix.A_log": (H,),
+                        p + "mix.dt_bias": (H,), p + "mix.norm": (dv,)})
+        else:
+            r = m["kv_rank"]
+            out.update({p + "mix.dkv": (r, W), p + "mix.dkv.norm": (r,), p + "mix.uk": (H * dk, r), p + "mix.uv": (H * dv, r),
+                        p + "mix.sink": (H,)})
+        if layer["mlp"] is not None:
+            F = layer["mlp"]["ff"]
+            out.update({p + "norm2": (W,), p + "mlp.gate": (F, W), p + "mlp.up": (F, W), p + "mlp.down": (W, F)})
+    return out
+
+
+def zuselix_tensor(name: str, shape: tuple, rng) -> np.ndarray:
+    """one tensor's random fp32 values: unit-variance sums, norm weights around 1, decays and steps of a few tokens to hundreds"""
+    last = name.rsplit(".", 1)[-1]
+    if last == "A_log":
+        return np.log(rng.uniform(0.05, 2.0, shape)).astype(np.float32)
+    a = rng.standard_normal(shape, dtype=np.float32)
+    if "norm" in last:
+        return 1.0 + 0.2 * a
+    if last == "dt_bias":
+        return a - 2.0
+    if last == "sink":
+        return 1.5 * a
+    if last == "conv":
+        return 0.6 * a
+    return a if name == "embed" else a / np.float32(np.sqrt(shape[-1]))
+
+
 def prompt(vocab: int, length: int = 16, seed: int = 0) -> list:
     rng = np.random.default_rng(seed + 1000)
     return [int(t) for t in rng.integers(0, vocab, size=length)]

@@ -125,4 +125,4 @@ def zuselix(config, tensors, tokens):
         stream.append(x)
     logits = layer_norm(x, t["final.norm"], eps) @ t["head"].T
     cap = config["logit_softcap"]
-    return cap * np.tanh(logits / cap), np.array(stream)
+    return cap * np.tanh(logits / cap) if cap else logits, np.array(stream)

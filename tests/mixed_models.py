@@ -2,7 +2,7 @@
 whose values bf16 holds exactly."""
 import numpy as np
 
-from caten_amd import llm
+from caten_amd import llm, synth
 from caten_amd.quant import from_bf16, to_bf16
 
 
@@ -22,52 +22,16 @@ def config(layers, width=128, vocab=320, eps=1e-5, cap=20.0):
     return {"architecture": "Zuselix", "layers": layers, "logit_softcap": cap, "norm": {"eps": eps}, "vocab": vocab, "width": width}
 
 
-def shapes(cfg):
-    W, V = cfg["width"], cfg["vocab"]
-    out = {"embed": (V, W), "final.norm": (W,), "head": (V, W)}
-    for i, l in enumerate(cfg["layers"]):
-        m, p = l["mixer"], f"l{i}."
-        out[p + "norm1"] = (W,)
-        H, dk, dv = m["heads"], m["dim"], m["vdim"]
-        if l["type"] == "delta":
-            K, n = m["kv_heads"] * dk, m["conv"]
-            out.update({p + "mix.q": (K, W), p + "mix.q.conv": (K, n), p + "mix.k": (K, W), p + "mix.k.conv": (K, n),
-                        p + "mix.v": (H * dv, W), p + "mix.v.conv": (H * dv, n), p + "mix.b": (H, W), p + "mix.a": (H, W),
-                        p + "mix.A_log": (H,), p + "mix.dt_bias": (H,), p + "mix.norm": (dv,), p + "mix.g": (H * dv, W),
-                        p + "mix.o": (W, H * dv)})
-        else:
-            r = m["kv_rank"]
-            out.update({p + "mix.q": (H * dk, W), p + "mix.dkv": (r, W), p + "mix.dkv.norm": (r,), p + "mix.uk": (H * dk, r),
-                        p + "mix.uv": (H * dv, r), p + "mix.sink": (H,), p + "mix.g": (H * dv, W), p + "mix.o": (W, H * dv)})
-        if l["mlp"] is not None:
-            F = l["mlp"]["ff"]
-            out.update({p + "norm2": (W,), p + "mlp.gate": (F, W), p + "mlp.up": (F, W), p + "mlp.down": (W, F)})
-    return out
-
-
 def weights(cfg, seed=0, **scale):
     """name -> fp32 array of bf16 values; scale: factor per tensor-name suffix"""
     rng = np.random.default_rng(seed)
     out = {}
-    for name, shape in shapes(cfg).items():
-        a = rng.standard_normal(shape)
-        last = name.rsplit(".", 1)[-1]
-        if "norm" in last:
-            a = 1.0 + 0.2 * a
-        elif last == "A_log":
-            a = np.log(rng.uniform(0.05, 2.0, shape))
-        elif last == "dt_bias":
-            a = a - 2.0
-        elif last == "sink":
-            a = 1.5 * a
-        elif last == "conv":
-            a = a * 0.6
-        elif name != "embed":
-            a = a / np.sqrt(shape[-1])
+    for name, shape in synth.zuselix_shapes(cfg).items():
+        a = synth.zuselix_tensor(name, shape, rng)
         for suffix, f in scale.items():
             if name.endswith("." + suffix):
                 a = a * f
-        out[name] = from_bf16(to_bf16(a.astype(np.float32).ravel())).reshape(shape)
+        out[name] = from_bf16(to_bf16(np.asarray(a, np.float32).ravel())).reshape(shape)
     return out
 
 
