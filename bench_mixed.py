@@ -123,23 +123,27 @@ def measure(name: str, kind: str, max_seq: int = 2304, prompts=(512, 2048), cont
     return res
 
 
-def main(names=None, kinds=("zuselix", "llama")) -> None:
+def main(names=None, kinds=("zuselix", "llama"), **measured) -> None:
     from caten_amd import synth
     for name in names or list(synth.ZUSELIX_CONFIGS):
         if name not in synth.ZUSELIX_CONFIGS:
             raise SystemExit(f"bench_mixed: unknown size {name} (known: {', '.join(synth.ZUSELIX_CONFIGS)})")
         for kind in kinds:
-            print(json.dumps(measure(name, kind)), flush=True)
+            print(json.dumps(measure(name, kind, **measured)), flush=True)
 
 
 if __name__ == "__main__":
     ap = argparse.ArgumentParser()
     ap.add_argument("--sizes", default="")
     ap.add_argument("--kinds", default="zuselix,llama")
+    ap.add_argument("--contexts", default="16,1900", help="prompt lengths in front of the timed decode steps")
+    ap.add_argument("--prompts", default="512,2048", help="timed prompt lengths")
+    ap.add_argument("--steps", type=int, default=64)
     ap.add_argument("--option", action="append", default=[], metavar="NAME=VALUE")
     a = ap.parse_args()
     from caten_amd import _lib
     for kv in a.option:
         opt, value = kv.split("=")
         _lib.check(_lib.init().cthip_set_option(opt.encode(), int(value)))
-    main([n for n in a.sizes.split(",") if n], a.kinds.split(","))
+    main([n for n in a.sizes.split(",") if n], a.kinds.split(","), steps=a.steps,
+         contexts=[int(c) for c in a.contexts.split(",") if c], prompts=[int(c) for c in a.prompts.split(",") if c])

@@ -173,7 +173,8 @@ static int load_latent(Decoder *d, int l) {
     DEC_TRY(to_f32(d, mkey(l, "mix.sink"), H, &v));
     a.sink = v;
   }
-  DEC_TRY(dev_alloc(d, (void **)&a.cache, sizeof(float) * (size_t)d->cfg.max_seq * a.R));
+  a.rows = d->cfg.max_seq;
+  DEC_TRY(dev_alloc(d, (void **)&a.cache, sizeof(float) * (size_t)a.rows * a.R));
   return 0;
 }
 
@@ -209,8 +210,7 @@ int mixed_load(Decoder *d) {
       DEC_TRY(to_f32(d, mkey(l, "norm2"), D, &L.norm2));
       RawTensor *g = nullptr;
       DEC_TRY(raw_of(d, mkey(l, "mlp.gate"), sp.ffn, D, &g));
-      // (a folded LayerNorm goes with row pairs only where a wavefront holds two rows at once)
-      L.fc_pairs = gemv_pair_swiglu_ok(g->type, 2 * (int64_t)sp.ffn, D) && (!ln || gemv_rows_per_wave(g->type, D) >= 2);
+      L.fc_pairs = gemv_pair_swiglu_ok(g->type, 2 * (int64_t)sp.ffn, D, ln);
       DEC_TRY(to_wmat(d, {mkey(l, "mlp.gate"), mkey(l, "mlp.up")}, 2 * (int64_t)sp.ffn, D, &L.gate_up, L.fc_pairs));
       DEC_TRY(to_wmat(d, {mkey(l, "mlp.down")}, D, sp.ffn, &L.down));
       if (ln) DEC_TRY(make_fold(d, L.gate_up, L.norm2, nullptr, nullptr, &L.fc_s, &none));

@@ -402,7 +402,7 @@ __device__ __forceinline__ void gemv_ring(const GemvArgs &a, float *xs_lds, floa
   // and the one after it; a slot's next tile is PD * total_waves further on either way.
   // (PAIR1 is its own instantiation: the others keep the plain order as constants)
   constexpr bool pair1 = PAIR1;
-  static_assert(!PAIR1 || (RPW == 1 && PD >= 2 && PD % 2 == 0 && !EPI && !DIRECT), "row pairs in ring slots: one row per wavefront, an even ring");
+  static_assert(!PAIR1 || (RPW == 1 && PD >= 2 && PD % 2 == 0 && !EPI), "row pairs in ring slots: one row per wavefront, an even ring");
   const int first = pair1 ? 2 * wave : wave;
   auto slot_off = [&](int p) { return pair1 ? (p >> 1) * 2 * total_waves + (p & 1) : p * total_waves; };
   const int own = first < nrq ? first : nrq - 1;  // what a slot without a tile requests: lines this wavefront fetches anyway
@@ -812,6 +812,7 @@ struct GemvVariant {
   gemv_fn fn_epi[2];   // the same with per-row epilogue operands (bias, residual, fold term) travelling in the ring
   gemv_fn fn_direct[2];  // looping, no epilogue operands, a LayerNorm applied to the staged input
   gemv_fn fn_small[2]; // one tile per wavefront: latency-bound launches
+  gemv_fn fn_pair_direct[2];  // the next with a LayerNorm applied to the staged input (bf16, fp16 and fp32 weights)
   gemv_fn fn_pair[2];  // looping, one row per wavefront, (gate, up) row pairs in neighbouring ring slots with SwiGLU as the epilogue; null where the shape has none
 };
 template <int T, int G, int KC, bool NT>
@@ -819,11 +820,18 @@ constexpr gemv_fn gemv_pair_fn() {
   if constexpr (G == 64 && PD_OF_T(T, KC) >= 2 && PD_OF_T(T, KC) % 2 == 0) return k_gemv<T, G, KC, PD_OF_T(T, KC), NT, false, false, true>;
   else return nullptr;
 }
+template <int T, int G, int KC, bool NT>
+constexpr gemv_fn gemv_pair_direct_fn() {
+  if constexpr (T != CTHIP_Q8_0 && T != CTHIP_Q4_0 && G == 64 && PD_OF_T(T, KC) >= 2 && PD_OF_T(T, KC) % 2 == 0)
+    return k_gemv<T, G, KC, PD_OF_T(T, KC), NT, false, true, true>;
+  else return nullptr;
+}
 #define V(T, G, KC)                                                                           \
   {T, G, KC, {k_gemv<T, G, KC, PD_OF_T(T, KC), false>, k_gemv<T, G, KC, PD_OF_T(T, KC), true>},         \
    {k_gemv<T, G, KC, PD_OF_T(T, KC), false, PD_OF_T(T, KC) != 1>, k_gemv<T, G, KC, PD_OF_T(T, KC), true, PD_OF_T(T, KC) != 1>}, \
    {k_gemv<T, G, KC, PD_OF_T(T, KC), false, false, PD_OF_T(T, KC) != 1>, k_gemv<T, G, KC, PD_OF_T(T, KC), true, false, PD_OF_T(T, KC) != 1>}, \
    {k_gemv<T, G, KC, 1, false>, k_gemv<T, G, KC, 1, true>},                                              \
+   {gemv_pair_direct_fn<T, G, KC, false>(), gemv_pair_direct_fn<T, G, KC, true>()},                      \
    {gemv_pair_fn<T, G, KC, false>(), gemv_pair_fn<T, G, KC, true>()}},
 // defined in gemv_q8.hip, gemv_q4.hip, gemv_f32.hip, gemv_f16.hip, gemv_bf16.hip
 extern const GemvVariant kGemvQ8[], kGemvQ4[], kGemvF32[], kGemvF16[], kGemvBF16[];

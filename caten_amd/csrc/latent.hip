@@ -84,17 +84,9 @@ __global__ __launch_bounds__(256) void k_latent_absorb(LatentArgs a, float *__re
   if (l == 0) qa[row] = v * a.scale;
 }
 
-// How the visible rows are cut: tiles of 16, `per` tiles to a range, `used` ranges not empty.
-struct LatentCut {
-  int per, used;
-};
-__device__ __forceinline__ LatentCut latent_cut(int T, int ranges) {
-  const int tiles = (T + 15) >> 4;
-  LatentCut c;
-  c.per = (tiles + ranges - 1) / ranges;
-  c.used = (tiles + c.per - 1) / c.per;
-  return c;
-}
+// The visible rows are tiles of 16; range r takes tiles r, r + ranges, ...: its first tile does not depend on how many rows
+// there are.  Ranges 0 .. latent_used() - 1 hold at least one row.
+__device__ __forceinline__ int latent_used(int T, int ranges) { return min((T + 15) >> 4, ranges); }
 
 // Workgroup (range, group of 16 heads), four wavefronts.
 //   S^T = C Q^T: a wavefront takes every fourth 16-float piece of the latent; lane l feeds C[key l%16] and Q[head l%16] with
@@ -109,10 +101,7 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentArgs a, const float
   __shared__ float sx[2][4][4][64];
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, lo = lane & 15, hi = lane >> 4;
   const int range = blockIdx.x, h0 = blockIdx.y * 16, R = a.R, H = a.H;
-  const int T = pos[0] + 1;
-  const LatentCut cut = latent_cut(T, ranges);
-  if (range >= cut.used) return;
-  const int tile0 = range * cut.per, tile1 = min(tile0 + cut.per, (T + 15) >> 4);
+  const int last = a.rows - 1;  // of the cache; rows past the visible ones are masked
   const int np = R >> 4, hq = min(h0 + lo, H - 1);  // heads past the end repeat the last one and are not stored
   constexpr int NP = 4 * NB;                        // pieces per wavefront, at most
   float4 q[NP];
@@ -129,13 +118,26 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentArgs a, const float
   float m = -INFINITY, L = 0.0f;
   float4 kc[NP];
   auto load_k = [&](int tile) {
-    const float *row = a.cache + (int64_t)min(tile * 16 + lo, T - 1) * R;
+    const float *row = a.cache + (int64_t)min(tile * 16 + lo, last) * R;
 #pragma unroll
     for (int i = 0; i < NP; i++) kc[i] = *(const float4 *)(row + 16 * min(wv + 4 * i, np - 1) + 4 * hi);  // (past the end: times zeros)
   };
-  load_k(tile0);
-  for (int tile = tile0; tile < tile1; tile++) {
-    const int kb = tile * 16, buf = tile & 1;
+  float4 vc[NB][4];
+  auto load_v = [&](int tile) {
+#pragma unroll
+    for (int b = 0; b < NB; b++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int e = min(64 * (wv + 4 * b) + 4 * lo, R - 4);  // (past the end: results are not stored)
+        vc[b][i] = *(const float4 *)(a.cache + (int64_t)min(tile * 16 + 4 * hi + i, last) * R + e);
+      }
+  };
+  load_k(range);
+  load_v(range);
+  const int T = pos[0] + 1, tiles = (T + 15) >> 4;
+  int buf = 0;
+  for (int tile = range; tile < tiles; tile += ranges, buf ^= 1) {
+    const int kb = tile * 16, next = tile + ranges < tiles ? tile + ranges : tile;
     v4f_t s = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int i = 0; i < NP; i++) {
@@ -144,16 +146,15 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentArgs a, const float
       s = __builtin_amdgcn_mfma_f32_16x16x4f32(kc[i].z, q[i].z, s, 0, 0, 0);
       s = __builtin_amdgcn_mfma_f32_16x16x4f32(kc[i].w, q[i].w, s, 0, 0, 0);
     }
-    // the rows as values, and the next tile's keys
-    float4 vc[NB][4];
+    load_k(next);
+    if (kb + 16 > T) {  // (rows no token has written yet, or an earlier sequence: their weight is zero, their values need not be numbers)
 #pragma unroll
-    for (int b = 0; b < NB; b++)
+      for (int i = 0; i < 4; i++)
+        if (kb + 4 * hi + i >= T) {
 #pragma unroll
-      for (int i = 0; i < 4; i++) {
-        const int e = min(64 * (wv + 4 * b) + 4 * lo, R - 4);  // (past the end: results are not stored)
-        vc[b][i] = *(const float4 *)(a.cache + (int64_t)min(kb + 4 * hi + i, T - 1) * R + e);
-      }
-    load_k(min(tile + 1, tile1 - 1));
+          for (int b = 0; b < NB; b++) vc[b][i] = make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+    }
 #pragma unroll
     for (int i = 0; i < 4; i++) sx[buf][wv][i][lane] = s[i];
     __syncthreads();  // (two buffers: the next tile's writes do not meet this tile's reads)
@@ -190,8 +191,9 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentArgs a, const float
         o[b][3] = __builtin_amdgcn_mfma_f32_16x16x4f32(vc[b][i].w, sc[i], o[b][3], 0, 0, 0);
       }
     }
+    load_v(next);
   }
-  if (h0 + lo < H) {
+  if (range < tiles && h0 + lo < H) {
     float *dst = part + ((int64_t)range * H + h0 + lo) * (R + 2);
 #pragma unroll
     for (int b = 0; b < NB; b++)
@@ -214,21 +216,32 @@ template <int TYPE>
 __global__ __launch_bounds__(256) void k_latent_up(LatentArgs a, const float *__restrict__ part, float *__restrict__ out,
                                                    const int *__restrict__ pos, int ranges) {
   extern __shared__ float x[];  // R floats
+  __shared__ float wr[kLatentMaxRanges];
   const int h = blockIdx.x, R = a.R, tid = threadIdx.x, l = tid & 15;
-  const LatentCut cut = latent_cut(pos[0] + 1, ranges);
   const float *__restrict__ ph = part + (int64_t)h * (R + 2);
   const int64_t pitch = (int64_t)a.H * (R + 2);
   const float sink = a.sink ? a.sink[h] : -INFINITY;
-  float M = sink;
-  for (int r = 0; r < cut.used; r++) M = fmaxf(M, ph[r * pitch + R]);
-  float L = expf(sink - M);
-  for (int r = 0; r < cut.used; r++) L = fmaf(expf(ph[r * pitch + R] - M), ph[r * pitch + R + 1], L);
-  const float inv = 1.0f / L;
+  const int used = latent_used(pos[0] + 1, ranges);
+  // the first wavefront: a range per lane, its weight in the merged softmax
+  if (tid < 64) {
+    const int r = min(tid, used - 1);
+    const float m = ph[r * pitch + R], d = tid < used ? ph[r * pitch + R + 1] : 0.0f;
+    const float M = fmaxf(wave_max(m), sink);
+    const float e = expf(m - M);
+    const float L = wave_sum(e * d) + expf(sink - M);  // (every lane takes part in the sum)
+    wr[tid] = tid < used ? e / L : 0.0f;
+  }
+  __syncthreads();
   for (int i = tid; i < R; i += 256) {
     float acc = 0.0f;
-#pragma unroll 8
-    for (int r = 0; r < cut.used; r++) acc = fmaf(expf(ph[r * pitch + R] - M), ph[r * pitch + i], acc);
-    x[i] = acc * inv;
+    for (int r0 = 0; r0 < used; r0 += 16) {  // sixteen requests together
+      float t[16];
+#pragma unroll
+      for (int k = 0; k < 16; k++) t[k] = ph[min(r0 + k, used - 1) * pitch + i];
+#pragma unroll
+      for (int k = 0; k < 16; k++) acc = fmaf(r0 + k < used ? wr[(r0 + k) & (kLatentMaxRanges - 1)] : 0.0f, t[k], acc);
+    }
+    x[i] = acc;
   }
   __syncthreads();
   for (int j = blockIdx.y * 16 + (tid >> 4); j < a.DV; j += 16 * gridDim.y) {

@@ -391,15 +391,18 @@ static bool gemv_prefers_wide(const GemvVariant *v, int type, int64_t rows) {
   const int opt = state().gemv_wide;
   return opt && (!v || heavy || opt >= 2);
 }
-bool gemv_pair_swiglu_ok(int type, int64_t rows, int64_t cols) {
+bool gemv_pair_swiglu_ok(int type, int64_t rows, int64_t cols, bool layernorm) {
   if (rows <= 0 || (rows & 1) || cols <= 0 || cols > 0x7fffffff) return false;
   const GemvVariant *v = pick_variant(type, (int)cols);
   const State &s = state();
-  if (gemv_prefers_wide(v, type, rows)) {
+  if (!layernorm && gemv_prefers_wide(v, type, rows)) {
     const GemvWidePlan p = gemv_wide_plan(type, rows, cols, s.compute_units);
     if (p.ok) return p.rw == 2;
   }
   if (!v) return false;
+  // one row per wavefront and a LayerNorm: only launches that normalise while they stage (gemv_plan) have no per-row
+  // operands in the ring
+  if (layernorm && v->G > 32 && (cols < 2048 || cols > 4096 || !v->fn_pair_direct[0])) return false;
   if (v->G <= 32) return true;  // two rows and more per wavefront: the pair sits in neighbouring lane groups
   // one row per wavefront: the pair sits in neighbouring slots of the ring, which a looping launch with an even ring
   // has (enough rows for every wavefront to loop at any occupancy)
@@ -457,7 +460,8 @@ static int launch_variant(const GemvVariant *v, const WMat *w, GemvArgs a, int m
     if (p.error) return fail(CTHIP_E_UNSUPPORTED, "gemv: (%d, %d): %s", a.rows, a.cols, p.error);
     // the paired SwiGLU epilogue with one row per wavefront: the pair sits in two neighbouring slots of the ring
     const bool pair1 = a.pair_swiglu && v->G > 32;
-    if (pair1 && (p.kernel != GEMV_K_LOOP || !v->fn_pair[0]))
+    const bool pair_direct = pair1 && p.kernel == GEMV_K_LOOP_DIRECT;
+    if (pair1 && (pair_direct ? !v->fn_pair_direct[0] : p.kernel != GEMV_K_LOOP || !v->fn_pair[0]))
       return fail(CTHIP_E_UNSUPPORTED, "gemv: the paired SwiGLU epilogue over (%d, %d) needs a looping launch with an even ring and no per-row operands", a.rows, a.cols);
     a.stage_x = p.stage ? 1 : 0;
     if (p.unfold) {
@@ -470,7 +474,7 @@ static int launch_variant(const GemvVariant *v, const WMat *w, GemvArgs a, int m
     // the looping kernel with per-row operands in its ring dereferences one of them unconditionally
     if (p.kernel == GEMV_K_LOOP_EPI && !a.bias && !a.residual && !a.fold_s)
       return fail(CTHIP_E_STATE, "gemv: a launch with epilogue operands in its ring has none");
-    const gemv_fn fn = pair1 ? v->fn_pair[nt] : p.kernel == GEMV_K_SMALL ? v->fn_small[nt] : p.kernel == GEMV_K_LOOP_EPI ? v->fn_epi[nt]
+    const gemv_fn fn = pair_direct ? v->fn_pair_direct[nt] : pair1 ? v->fn_pair[nt] : p.kernel == GEMV_K_SMALL ? v->fn_small[nt] : p.kernel == GEMV_K_LOOP_EPI ? v->fn_epi[nt]
                      : p.kernel == GEMV_K_LOOP_DIRECT ? v->fn_direct[nt] : v->fn[nt];
     hipLaunchKernelGGL(fn, dim3(p.grid_x, p.grid_y), dim3(p.block), p.lds, s.stream, a);
     CTHIP_LAUNCH_CHECK();

@@ -40,7 +40,8 @@ struct LatentArgs {
   const float *norm;   // [R], zeros in the padding
   int gated;           // the output is multiplied by sigmoid(g)
   const float *sink;   // [H] logits of the extra softmax term (no key, no value); null = none
-  float *cache;        // [max_seq][R]
+  float *cache;        // [rows][R]
+  int rows;
   int type;            // weight type of absorb / up
   const void *absorb;  // [H][R][DK]: the key projection, transposed per head
   const void *up;      // [H][DV][R]: the value projection
