@@ -48,12 +48,25 @@ __device__ __forceinline__ float row_dot16(const void *__restrict__ w, int64_t r
   return acc;
 }
 
-// a wavefront normalises one latent
+// a wavefront normalises one latent (R <= 1024); everything is requested before anything is used
 __device__ __forceinline__ void latent_norm(const LatentArgs &a, const float *__restrict__ src, float *__restrict__ dst, int lane) {
+  float4 x[4], w[4];
   float ss = 0.0f;
-  for (int i = lane; i < a.R; i += 64) ss = fmaf(src[i], src[i], ss);  // padding entries are zero
+#pragma unroll
+  for (int k = 0; k < 4; k++) {
+    const int e = min(4 * (lane + 64 * k), a.R - 4);
+    x[k] = *(const float4 *)(src + e);
+    w[k] = *(const float4 *)(a.norm + e);
+  }
+#pragma unroll
+  for (int k = 0; k < 4; k++)
+    if (4 * (lane + 64 * k) < a.R) ss = fmaf(x[k].x, x[k].x, fmaf(x[k].y, x[k].y, fmaf(x[k].z, x[k].z, fmaf(x[k].w, x[k].w, ss))));  // padding entries are zero
   const float rstd = 1.0f / sqrtf(wave_sum(ss) / (float)a.r + a.eps);
-  for (int i = lane; i < a.R; i += 64) dst[i] = src[i] * rstd * a.norm[i];
+#pragma unroll
+  for (int k = 0; k < 4; k++) {
+    const int e = 4 * (lane + 64 * k);
+    if (e < a.R) *(float4 *)(dst + e) = make_float4(x[k].x * rstd * w[k].x, x[k].y * rstd * w[k].y, x[k].z * rstd * w[k].z, x[k].w * rstd * w[k].w);
+  }
 }
 
 __global__ __launch_bounds__(256) void k_latent_append(LatentArgs a, int s, int n) {
@@ -88,80 +101,84 @@ __global__ __launch_bounds__(256) void k_latent_absorb(LatentArgs a, float *__re
 // there are.  Ranges 0 .. latent_used() - 1 hold at least one row.
 __device__ __forceinline__ int latent_used(int T, int ranges) { return min((T + 15) >> 4, ranges); }
 
-// Workgroup (range, group of 16 heads), four wavefronts.
+// Workgroup (range, group of 16 heads), four wavefronts.  A tile of 16 cached rows is fetched once, into LDS, a tile ahead.
 //   S^T = C Q^T: a wavefront takes every fourth 16-float piece of the latent; lane l feeds C[key l%16] and Q[head l%16] with
 //     the four floats 4 (l/16) .. of the piece (the same order on both sides), so it ends up with keys 4 (l/16) + i of head
 //     l % 16; the four wavefronts' sums meet in LDS;
 //   O^T += C^T P^T: a wavefront owns every fourth 64-float block of the latent; register i of a lane is exactly the
-//     probability that matrix instruction i wants from it, and the 16 bytes 4 (l%16) .. of cached row 4 (l/16) + i are its
+//     probability that matrix instruction i wants from it, and the 16 bytes 4 (l%16) .. of row 4 (l/16) + i of the tile are its
 //     operands for four output tiles (tile t: latent entry 64 b + 4 m + t in row m).
-template <int NB>  // 64-float blocks per wavefront
+constexpr int part_pitch(int R) { return R + 4; }  // a range's record of one head: R sums, maximum, denominator, two unused
+template <int NB>  // 256-float blocks of a latent
 __global__ __launch_bounds__(256) void k_latent_attend(LatentArgs a, const float *__restrict__ qa, float *__restrict__ part,
                                                        const int *__restrict__ pos, int ranges) {
-  __shared__ float sx[2][4][4][64];
+  extern __shared__ float tiles_lds[];  // two tiles of 16 rows, R + 4 floats apart
+  __shared__ float sx[4][4][64];
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, lo = lane & 15, hi = lane >> 4;
-  const int range = blockIdx.x, h0 = blockIdx.y * 16, R = a.R, H = a.H;
+  const int range = blockIdx.x, h0 = blockIdx.y * 16, R = a.R, H = a.H, LD = R + 4;
   const int last = a.rows - 1;  // of the cache; rows past the visible ones are masked
   const int np = R >> 4, hq = min(h0 + lo, H - 1);  // heads past the end repeat the last one and are not stored
   constexpr int NP = 4 * NB;                        // pieces per wavefront, at most
+  float4 pf[4][NB];  // rows 4 wv .. 4 wv + 3 of the tile that comes next
+  auto fetch = [&](int tile) {
+#pragma unroll
+    for (int r = 0; r < 4; r++) {
+      const float *row = a.cache + (int64_t)min(tile * 16 + 4 * wv + r, last) * R;
+#pragma unroll
+      for (int b = 0; b < NB; b++) pf[r][b] = *(const float4 *)(row + min(4 * (lane + 64 * b), R - 4));
+    }
+  };
+  fetch(range);  // (which tile a range starts with does not depend on the position)
+  const int T = pos[0] + 1, tiles = (T + 15) >> 4;
   float4 q[NP];
 #pragma unroll
   for (int i = 0; i < NP; i++) {
     const int pc = wv + 4 * i;
-    q[i] = pc < np ? *(const float4 *)(qa + (int64_t)hq * R + 16 * pc + 4 * hi) : make_float4(0.f, 0.f, 0.f, 0.f);
+    const float4 v = *(const float4 *)(qa + (int64_t)hq * R + 16 * min(pc, np - 1) + 4 * hi);
+    q[i] = pc < np ? v : make_float4(0.f, 0.f, 0.f, 0.f);
   }
+  if (range >= tiles) return;
+  auto put = [&](int tile, int buf) {  // rows that no token of this sequence has written are zeroed: their weight is zero, their values need not be numbers
+#pragma unroll
+    for (int r = 0; r < 4; r++) {
+      const bool seen = tile * 16 + 4 * wv + r < T;
+      float *row = tiles_lds + (buf * 16 + 4 * wv + r) * LD;
+#pragma unroll
+      for (int b = 0; b < NB; b++) {
+        const int e = 4 * (lane + 64 * b);
+        if (e < R) *(float4 *)(row + e) = seen ? pf[r][b] : make_float4(0.f, 0.f, 0.f, 0.f);
+      }
+    }
+  };
   v4f_t o[NB][4];
 #pragma unroll
   for (int b = 0; b < NB; b++)
 #pragma unroll
     for (int t = 0; t < 4; t++) o[b][t] = v4f_t{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, L = 0.0f;
-  float4 kc[NP];
-  auto load_k = [&](int tile) {
-    const float *row = a.cache + (int64_t)min(tile * 16 + lo, last) * R;
-#pragma unroll
-    for (int i = 0; i < NP; i++) kc[i] = *(const float4 *)(row + 16 * min(wv + 4 * i, np - 1) + 4 * hi);  // (past the end: times zeros)
-  };
-  float4 vc[NB][4];
-  auto load_v = [&](int tile) {
-#pragma unroll
-    for (int b = 0; b < NB; b++)
-#pragma unroll
-      for (int i = 0; i < 4; i++) {
-        const int e = min(64 * (wv + 4 * b) + 4 * lo, R - 4);  // (past the end: results are not stored)
-        vc[b][i] = *(const float4 *)(a.cache + (int64_t)min(tile * 16 + 4 * hi + i, last) * R + e);
-      }
-  };
-  load_k(range);
-  load_v(range);
-  const int T = pos[0] + 1, tiles = (T + 15) >> 4;
   int buf = 0;
+  put(range, 0);
+  fetch(min(range + ranges, tiles - 1));
+  __syncthreads();
   for (int tile = range; tile < tiles; tile += ranges, buf ^= 1) {
-    const int kb = tile * 16, next = tile + ranges < tiles ? tile + ranges : tile;
-    v4f_t s = {0.f, 0.f, 0.f, 0.f};
+    const int kb = tile * 16;
+    const float *Ct = tiles_lds + buf * 16 * LD;
+    v4f_t s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int i = 0; i < NP; i++) {
-      s = __builtin_amdgcn_mfma_f32_16x16x4f32(kc[i].x, q[i].x, s, 0, 0, 0);
-      s = __builtin_amdgcn_mfma_f32_16x16x4f32(kc[i].y, q[i].y, s, 0, 0, 0);
-      s = __builtin_amdgcn_mfma_f32_16x16x4f32(kc[i].z, q[i].z, s, 0, 0, 0);
-      s = __builtin_amdgcn_mfma_f32_16x16x4f32(kc[i].w, q[i].w, s, 0, 0, 0);
-    }
-    load_k(next);
-    if (kb + 16 > T) {  // (rows no token has written yet, or an earlier sequence: their weight is zero, their values need not be numbers)
-#pragma unroll
-      for (int i = 0; i < 4; i++)
-        if (kb + 4 * hi + i >= T) {
-#pragma unroll
-          for (int b = 0; b < NB; b++) vc[b][i] = make_float4(0.f, 0.f, 0.f, 0.f);
-        }
+      const float4 kc = *(const float4 *)(Ct + lo * LD + 16 * min(wv + 4 * i, np - 1) + 4 * hi);  // (past the end: times zeros)
+      s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(kc.x, q[i].x, s0, 0, 0, 0);
+      s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(kc.y, q[i].y, s1, 0, 0, 0);
+      s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(kc.z, q[i].z, s0, 0, 0, 0);
+      s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(kc.w, q[i].w, s1, 0, 0, 0);
     }
 #pragma unroll
-    for (int i = 0; i < 4; i++) sx[buf][wv][i][lane] = s[i];
-    __syncthreads();  // (two buffers: the next tile's writes do not meet this tile's reads)
+    for (int i = 0; i < 4; i++) sx[wv][i][lane] = s0[i] + s1[i];
+    __syncthreads();
     float sc[4], top = -INFINITY;
 #pragma unroll
     for (int i = 0; i < 4; i++) {
-      sc[i] = (sx[buf][0][i][lane] + sx[buf][1][i][lane]) + (sx[buf][2][i][lane] + sx[buf][3][i][lane]);
+      sc[i] = (sx[0][i][lane] + sx[1][i][lane]) + (sx[2][i][lane] + sx[3][i][lane]);
       if (kb + 4 * hi + i >= T) sc[i] = -INFINITY;
       top = fmaxf(top, sc[i]);
     }
@@ -181,76 +198,96 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentArgs a, const float
     m = m_new;
 #pragma unroll
     for (int b = 0; b < NB; b++) {
+      const float *vcol = Ct + 4 * hi * LD + min(64 * (wv + 4 * b) + 4 * lo, R - 4);  // (past the end: results are not stored)
 #pragma unroll
       for (int t = 0; t < 4; t++) o[b][t] *= corr;
 #pragma unroll
       for (int i = 0; i < 4; i++) {
-        o[b][0] = __builtin_amdgcn_mfma_f32_16x16x4f32(vc[b][i].x, sc[i], o[b][0], 0, 0, 0);
-        o[b][1] = __builtin_amdgcn_mfma_f32_16x16x4f32(vc[b][i].y, sc[i], o[b][1], 0, 0, 0);
-        o[b][2] = __builtin_amdgcn_mfma_f32_16x16x4f32(vc[b][i].z, sc[i], o[b][2], 0, 0, 0);
-        o[b][3] = __builtin_amdgcn_mfma_f32_16x16x4f32(vc[b][i].w, sc[i], o[b][3], 0, 0, 0);
+        const float4 vc = *(const float4 *)(vcol + i * LD);
+        o[b][0] = __builtin_amdgcn_mfma_f32_16x16x4f32(vc.x, sc[i], o[b][0], 0, 0, 0);
+        o[b][1] = __builtin_amdgcn_mfma_f32_16x16x4f32(vc.y, sc[i], o[b][1], 0, 0, 0);
+        o[b][2] = __builtin_amdgcn_mfma_f32_16x16x4f32(vc.z, sc[i], o[b][2], 0, 0, 0);
+        o[b][3] = __builtin_amdgcn_mfma_f32_16x16x4f32(vc.w, sc[i], o[b][3], 0, 0, 0);
       }
     }
-    load_v(next);
+    if (tile + ranges < tiles) {  // (uniform over the workgroup)
+      put(tile + ranges, buf ^ 1);
+      fetch(min(tile + 2 * ranges, tiles - 1));
+    }
+    __syncthreads();
   }
-  if (range < tiles && h0 + lo < H) {
-    float *dst = part + ((int64_t)range * H + h0 + lo) * (R + 2);
+  if (h0 + lo < H) {
+    float *dst = part + ((int64_t)range * H + h0 + lo) * part_pitch(R);
 #pragma unroll
     for (int b = 0; b < NB; b++)
 #pragma unroll
-      for (int t = 0; t < 4; t++)
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-          const int e = 64 * (wv + 4 * b) + 4 * (4 * hi + i) + t;
-          if (e < R) dst[e] = o[b][t][i];
-        }
-    if (wv == 0 && hi == 0) {
-      dst[R] = m;
-      dst[R + 1] = L;
-    }
+      for (int i = 0; i < 4; i++) {
+        const int e = 64 * (wv + 4 * b) + 4 * (4 * hi + i);
+        if (e < R) *(float4 *)(dst + e) = make_float4(o[b][0][i], o[b][1][i], o[b][2][i], o[b][3][i]);
+      }
+    if (wv == 0 && hi == 0) *(float2 *)(dst + R) = make_float2(m, L);
   }
 }
 
-// workgroup (head, share of its value rows): merged latent in LDS, then 16 lanes per value row
+// Workgroup (head, share of its value rows): the ranges merged in LDS, then 16 lanes per value row.  The ranges' sums are
+// requested before their weights are known; 256 / (R / 4) groups of threads share the ranges.
 template <int TYPE>
 __global__ __launch_bounds__(256) void k_latent_up(LatentArgs a, const float *__restrict__ part, float *__restrict__ out,
                                                    const int *__restrict__ pos, int ranges) {
-  extern __shared__ float x[];  // R floats
+  constexpr int AHEAD = 8;
+  extern __shared__ float x[];  // the groups' merged latents, R floats each
   __shared__ float wr[kLatentMaxRanges];
   const int h = blockIdx.x, R = a.R, tid = threadIdx.x, l = tid & 15;
-  const float *__restrict__ ph = part + (int64_t)h * (R + 2);
-  const int64_t pitch = (int64_t)a.H * (R + 2);
+  const float *__restrict__ ph = part + (int64_t)h * part_pitch(R);
+  const int64_t pitch = (int64_t)a.H * part_pitch(R);
+  const int n4 = R >> 2, ng = 256 / n4, grp = tid / n4, col = 4 * (tid - grp * n4);
+  const float2 ml = *(const float2 *)(ph + min(tid & 63, ranges - 1) * pitch + R);
+  float4 t[AHEAD];
+#pragma unroll
+  for (int k = 0; k < AHEAD; k++) t[k] = *(const float4 *)(ph + min(grp + ng * k, ranges - 1) * pitch + col);
   const float sink = a.sink ? a.sink[h] : -INFINITY;
   const int used = latent_used(pos[0] + 1, ranges);
-  // the first wavefront: a range per lane, its weight in the merged softmax
-  if (tid < 64) {
-    const int r = min(tid, used - 1);
-    const float m = ph[r * pitch + R], d = tid < used ? ph[r * pitch + R + 1] : 0.0f;
+  if (tid < 64) {  // the first wavefront: a range per lane, its weight in the merged softmax
+    const float m = tid < used ? ml.x : -INFINITY, d = tid < used ? ml.y : 0.0f;
     const float M = fmaxf(wave_max(m), sink);
     const float e = expf(m - M);
     const float L = wave_sum(e * d) + expf(sink - M);  // (every lane takes part in the sum)
-    wr[tid] = tid < used ? e / L : 0.0f;
+    wr[tid] = e / L;
   }
   __syncthreads();
-  for (int i = tid; i < R; i += 256) {
-    float acc = 0.0f;
-    for (int r0 = 0; r0 < used; r0 += 16) {  // sixteen requests together
-      float t[16];
+  if (grp < ng) {
+    float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+    auto add = [&](int r, const float4 v) {
+      if (r >= used) return;  // (what an unused range holds need not be numbers)
+      const float c = wr[r];
+      acc.x = fmaf(c, v.x, acc.x), acc.y = fmaf(c, v.y, acc.y), acc.z = fmaf(c, v.z, acc.z), acc.w = fmaf(c, v.w, acc.w);
+    };
 #pragma unroll
-      for (int k = 0; k < 16; k++) t[k] = ph[min(r0 + k, used - 1) * pitch + i];
+    for (int k = 0; k < AHEAD; k++) add(grp + ng * k, t[k]);
+    for (int r0 = grp + ng * AHEAD; r0 < used; r0 += ng * AHEAD) {
 #pragma unroll
-      for (int k = 0; k < 16; k++) acc = fmaf(r0 + k < used ? wr[(r0 + k) & (kLatentMaxRanges - 1)] : 0.0f, t[k], acc);
+      for (int k = 0; k < AHEAD; k++) t[k] = *(const float4 *)(ph + min(r0 + ng * k, used - 1) * pitch + col);
+#pragma unroll
+      for (int k = 0; k < AHEAD; k++) add(r0 + ng * k, t[k]);
     }
-    x[i] = acc;
+    *(float4 *)(x + grp * R + col) = acc;
   }
   __syncthreads();
+  if (ng > 1) {
+    for (int i = tid; i < R; i += 256) {
+      float v = x[i];
+      for (int g = 1; g < ng; g++) v += x[g * R + i];
+      x[i] = v;  // (read by this thread only until the barrier)
+    }
+    __syncthreads();
+  }
   for (int j = blockIdx.y * 16 + (tid >> 4); j < a.DV; j += 16 * gridDim.y) {
     const float v = row16_sum(row_dot16<TYPE>(a.up, (int64_t)h * a.DV + j, x, R, l));
     if (l == 0) out[h * a.DV + j] = a.gated ? v / (1.0f + expf(-a.p[(int64_t)a.H * a.DK + R + h * a.DV + j])) : v;
   }
 }
 
-size_t latent_part_floats(int H, int R, int ranges) { return (size_t)ranges * H * (R + 2); }
+size_t latent_part_floats(int H, int R, int ranges) { return (size_t)ranges * H * part_pitch(R); }
 
 int launch_latent_step(const LatentArgs &a, const LatentWork &w, float *out, const int *pos) {
   hipStream_t st = state().stream;
@@ -259,17 +296,28 @@ int launch_latent_step(const LatentArgs &a, const LatentWork &w, float *out, con
   int shares = state().compute_units / a.H;
   if (shares > a.DV / 16) shares = a.DV / 16;
   const dim3 gu((unsigned)a.H, (unsigned)(shares < 1 ? 1 : shares));
-  const size_t lds = sizeof(float) * (size_t)a.R;
+  const size_t lds = sizeof(float) * (size_t)a.R * (256 / (a.R / 4));
+  const size_t lds_tiles = sizeof(float) * 2 * 16 * (size_t)(a.R + 4);
   const int nb = (a.R + 255) / 256;
 #define ABSORB(T) hipLaunchKernelGGL((k_latent_absorb<T>), ga, dim3(256), 0, st, a, w.qa, pos)
 #define UP(T) hipLaunchKernelGGL((k_latent_up<T>), gu, dim3(256), lds, st, a, w.part, out, pos, w.ranges)
   if (a.type == CTHIP_BF16) ABSORB(CTHIP_BF16);
   else if (a.type == CTHIP_F16) ABSORB(CTHIP_F16);
   else ABSORB(CTHIP_F32);
-  if (nb <= 1) hipLaunchKernelGGL((k_latent_attend<1>), gt, dim3(256), 0, st, a, w.qa, w.part, pos, w.ranges);
-  else if (nb <= 2) hipLaunchKernelGGL((k_latent_attend<2>), gt, dim3(256), 0, st, a, w.qa, w.part, pos, w.ranges);
-  else if (nb <= 4) hipLaunchKernelGGL((k_latent_attend<4>), gt, dim3(256), 0, st, a, w.qa, w.part, pos, w.ranges);
+#define ATTEND(N)                                                                                                                       \
+  do {                                                                                                                                  \
+    static bool granted = false;                                                                                                        \
+    if (lds_tiles > 64 * 1024 && !granted) { /* once per kernel: more than the default share of LDS */                                  \
+      CTHIP_CHECK(hipFuncSetAttribute((const void *)k_latent_attend<N>, hipFuncAttributeMaxDynamicSharedMemorySize, 140 * 1024));         \
+      granted = true;                                                                                                                   \
+    }                                                                                                                                   \
+    hipLaunchKernelGGL((k_latent_attend<N>), gt, dim3(256), lds_tiles, st, a, w.qa, w.part, pos, w.ranges);                              \
+  } while (0)
+  if (nb <= 1) ATTEND(1);
+  else if (nb <= 2) ATTEND(2);
+  else if (nb <= 4) ATTEND(4);
   else return fail(CTHIP_E_UNSUPPORTED, "latent attention: a latent of %d (at most 1024)", a.R);
+#undef ATTEND
   if (a.type == CTHIP_BF16) UP(CTHIP_BF16);
   else if (a.type == CTHIP_F16) UP(CTHIP_F16);
   else UP(CTHIP_F32);

@@ -49,7 +49,7 @@ struct LatentArgs {
 constexpr int kLatentMaxRanges = 64;
 struct LatentWork {
   float *qa;    // [H][R]: queries carried into the latent space
-  float *part;  // [ranges][H][R + 2]: unnormalised sums, maximum, denominator of every key range
+  float *part;  // [ranges][H]: unnormalised sums, maximum and denominator of every key range (latent_part_floats)
   int ranges;
 };
 size_t latent_part_floats(int H, int R, int ranges);
