@@ -100,9 +100,10 @@ def prefill_ms(model, vocab: int, s: int):
     return min(ts) * 1e3
 
 
-def measure(name: str, kind: str, max_seq: int = 2304, prompts=(512, 2048), contexts=(16, 1900), steps: int = 64) -> dict:
+def measure(name: str, kind: str, prompts=(512, 2048), contexts=(16, 1900), steps: int = 64) -> dict:
     from caten_amd import _lib
     lib = _lib.init()
+    max_seq = max([c + steps + 16 for c in contexts] + list(prompts) + [64])
     t0 = time.perf_counter()
     model, cfg, gflop = (zuselix_session if kind == "zuselix" else llama_session)(name, max_seq)
     err = agree(model, cfg["vocab"])

@@ -97,9 +97,13 @@ __global__ __launch_bounds__(256) void k_latent_absorb(LatentArgs a, float *__re
   if (l == 0) qa[row] = v * a.scale;
 }
 
-// The visible rows are tiles of 16; range r takes tiles r, r + ranges, ...: its first tile does not depend on how many rows
-// there are.  Ranges 0 .. latent_used() - 1 hold at least one row.
-__device__ __forceinline__ int latent_used(int T, int ranges) { return min((T + 15) >> 4, ranges); }
+// The visible rows are tiles of 16; range r takes tiles r, r + n, ... of n ranges: its first tile does not depend on how many
+// rows there are.  A range's record is merged by every workgroup of k_latent_up, so up to four tiles go to a range before
+// more than 64 ranges are used (16 heads at position 1900: 32 / 64 ranges 954 / 942 us per step of the 1b shape).
+__device__ __forceinline__ int latent_ranges(int T, int most) {
+  const int tiles = (T + 15) >> 4;
+  return min(tiles, tiles > 256 ? most : min(most, 64));
+}
 
 // Workgroup (range, group of 16 heads), four wavefronts.  A tile of 16 cached rows is fetched once, into LDS, a tile ahead.
 //   S^T = C Q^T: a wavefront takes every fourth 16-float piece of the latent; lane l feeds C[key l%16] and Q[head l%16] with
@@ -137,7 +141,8 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentArgs a, const float
     const float4 v = *(const float4 *)(qa + (int64_t)hq * R + 16 * min(pc, np - 1) + 4 * hi);
     q[i] = pc < np ? v : make_float4(0.f, 0.f, 0.f, 0.f);
   }
-  if (range >= tiles) return;
+  const int nr = latent_ranges(T, ranges);  // every one of them holds at least one row
+  if (range >= nr) return;
   auto put = [&](int tile, int buf) {  // rows that no token of this sequence has written are zeroed: their weight is zero, their values need not be numbers
 #pragma unroll
     for (int r = 0; r < 4; r++) {
@@ -158,9 +163,9 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentArgs a, const float
   float m = -INFINITY, L = 0.0f;
   int buf = 0;
   put(range, 0);
-  fetch(min(range + ranges, tiles - 1));
+  fetch(min(range + nr, tiles - 1));
   __syncthreads();
-  for (int tile = range; tile < tiles; tile += ranges, buf ^= 1) {
+  for (int tile = range; tile < tiles; tile += nr, buf ^= 1) {
     const int kb = tile * 16;
     const float *Ct = tiles_lds + buf * 16 * LD;
     v4f_t s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
@@ -210,9 +215,9 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentArgs a, const float
         o[b][3] = __builtin_amdgcn_mfma_f32_16x16x4f32(vc.w, sc[i], o[b][3], 0, 0, 0);
       }
     }
-    if (tile + ranges < tiles) {  // (uniform over the workgroup)
-      put(tile + ranges, buf ^ 1);
-      fetch(min(tile + 2 * ranges, tiles - 1));
+    if (tile + nr < tiles) {  // (uniform over the workgroup)
+      put(tile + nr, buf ^ 1);
+      fetch(min(tile + 2 * nr, tiles - 1));
     }
     __syncthreads();
   }
@@ -241,18 +246,22 @@ __global__ __launch_bounds__(256) void k_latent_up(LatentArgs a, const float *__
   const float *__restrict__ ph = part + (int64_t)h * part_pitch(R);
   const int64_t pitch = (int64_t)a.H * part_pitch(R);
   const int n4 = R >> 2, ng = 256 / n4, grp = tid / n4, col = 4 * (tid - grp * n4);
-  const float2 ml = *(const float2 *)(ph + min(tid & 63, ranges - 1) * pitch + R);
+  float2 ml[2];
+#pragma unroll
+  for (int k = 0; k < 2; k++) ml[k] = *(const float2 *)(ph + min((tid & 63) + 64 * k, ranges - 1) * pitch + R);
   float4 t[AHEAD];
 #pragma unroll
   for (int k = 0; k < AHEAD; k++) t[k] = *(const float4 *)(ph + min(grp + ng * k, ranges - 1) * pitch + col);
   const float sink = a.sink ? a.sink[h] : -INFINITY;
-  const int used = latent_used(pos[0] + 1, ranges);
-  if (tid < 64) {  // the first wavefront: a range per lane, its weight in the merged softmax
-    const float m = tid < used ? ml.x : -INFINITY, d = tid < used ? ml.y : 0.0f;
-    const float M = fmaxf(wave_max(m), sink);
-    const float e = expf(m - M);
-    const float L = wave_sum(e * d) + expf(sink - M);  // (every lane takes part in the sum)
-    wr[tid] = e / L;
+  const int used = latent_ranges(pos[0] + 1, ranges);
+  if (tid < 64) {  // the first wavefront: two ranges per lane, their weights in the merged softmax
+    const float m0 = tid < used ? ml[0].x : -INFINITY, d0 = tid < used ? ml[0].y : 0.0f;
+    const float m1 = tid + 64 < used ? ml[1].x : -INFINITY, d1 = tid + 64 < used ? ml[1].y : 0.0f;
+    const float M = fmaxf(wave_max(fmaxf(m0, m1)), sink);
+    const float e0 = expf(m0 - M), e1 = expf(m1 - M);
+    const float L = wave_sum(e0 * d0 + e1 * d1) + expf(sink - M);  // (every lane takes part in the sum)
+    wr[tid] = e0 / L;
+    wr[tid + 64] = e1 / L;
   }
   __syncthreads();
   if (grp < ng) {

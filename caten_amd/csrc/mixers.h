@@ -46,7 +46,7 @@ struct LatentArgs {
   const void *absorb;  // [H][R][DK]: the key projection, transposed per head
   const void *up;      // [H][DV][R]: the value projection
 };
-constexpr int kLatentMaxRanges = 64;
+constexpr int kLatentMaxRanges = 128;
 struct LatentWork {
   float *qa;    // [H][R]: queries carried into the latent space
   float *part;  // [ranges][H]: unnormalised sums, maximum and denominator of every key range (latent_part_floats)
