@@ -367,9 +367,9 @@ int mixed_prefill(Decoder *d, float *X, float *XN, int s, int n) {
         r.S = s;
         r.start_pos = n;
         r.H = r.Hkv = a.H;
-        r.ldq = r.ldg = a.ldp;
-        r.ldk = r.ldv = L.kv_up->rows;
-        r.ldo = L.out->cols;
+        r.ldq = r.ldg = (int)a.ldp;
+        r.ldk = r.ldv = (int)L.kv_up->rows;
+        r.ldo = (int)L.out->cols;
         r.dk = a.DK;
         r.dv = a.DV;
         r.scale = a.scale;

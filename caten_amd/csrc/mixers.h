@@ -63,7 +63,7 @@ struct AttnRowsArgs {
   float *out;             // (S, H x dv), ldo floats apart
   const float *q, *k, *v; // rows ldq / ldk / ldv floats apart, heads dk / dk / dv floats apart
   int S, start_pos, H, Hkv;
-  int64_t ldq, ldk, ldv, ldo, ldg;
+  int ldq, ldk, ldv, ldo, ldg;
   int dk, dv;             // multiples of 4, at most 256
   float scale;
   const float *sink;      // [H] or null

@@ -1060,7 +1060,7 @@ int launch_attn(float *out, const float *q, const float *kc, const float *vc, in
     AttnRowsArgs rows = {};
     rows.out = out, rows.q = q, rows.k = kc, rows.v = vc;
     rows.S = S, rows.start_pos = start_pos, rows.H = H, rows.Hkv = Hkv;
-    rows.ldq = rows.ldo = (int64_t)H * Dh, rows.ldk = rows.ldv = (int64_t)Hkv * Dh;
+    rows.ldq = rows.ldo = H * Dh, rows.ldk = rows.ldv = Hkv * Dh;
     rows.dk = rows.dv = Dh;
     rows.scale = 1.0f / sqrtf((float)Dh);
     if (state().gemm_precision == 0) {  // fp32 operands asked for: the products are fp32 products

@@ -383,3 +383,39 @@ def test_bf16_linear(cols):
                 _lib.check(lib.cthip_set_option(b"gemm_precision", 2))
             assert np.abs(got - want).max() / np.sqrt((want ** 2).mean()) < tol, (m, prec)
     h.free()
+
+
+def test_what_a_mixed_decoder_refuses():
+    from caten_amd import _lib, llm
+    from caten_amd._lib import HipError
+    cfg = MODELS["latent"]
+    w = mm.weights(cfg, 20)
+    for layer, msg in ((mm.delta(dim=264), "at most 256"), (mm.delta(3, 2), "bad argument"), (mm.latent(kv_rank=1040), "at most 1024"),
+                       (mm.delta(conv=0), "bad argument")):
+        with pytest.raises(HipError, match=msg):
+            mm.session(mm.config([layer]), {})
+    short = dict(w)
+    del short["l0.mix.uk"]
+    with pytest.raises(HipError, match="1 tensors of the model are missing"):
+        mm.session(cfg, short)
+    with pytest.raises(HipError, match="not a tensor of this model"):
+        mm.session(cfg, dict(w, extra=w["embed"]))
+    m = mm.session(cfg, dict(w, **{"l0.mix.uk": w["l0.mix.uk"][:, :40]}))
+    with pytest.raises(HipError, match="l0.mix.uk.*expected"):
+        m.forward([1], 1, 0)
+    m.close()
+    sd = llm.safetensors_state_dict(mm.raw_tensors(w))
+    sd["l0.mix.dkv"] = llm.Tensor.from_f32(w["l0.mix.dkv"], "f32")
+    m = llm.MixedTransformer(dict(llm.zuselix_config(cfg), max_seq=16)).load_state_dict(sd)
+    with pytest.raises(HipError, match="its neighbours"):
+        m.forward([1], 1, 0)
+    m.close()
+    lib = _lib.init()
+    _lib.check(lib.cthip_set_option(b"kv_cache", 1))
+    try:
+        m = mm.session(cfg, w)
+        with pytest.raises(HipError, match="fp32 rows"):
+            m.forward([1], 1, 0)
+        m.close()
+    finally:
+        _lib.check(lib.cthip_set_option(b"kv_cache", 0))
