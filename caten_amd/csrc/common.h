@@ -130,8 +130,14 @@ struct AttnSplit;
 int launch_attn_q8_step(float *out, const float *q, const float *newkv, void *kq, void *kd, void *vq, void *vd, const int *pos,
                         int H, int Hkv, int Dh, float rope_base, const AttnSplit *split);
 
+// A gated unit of two projections: min(g, limit) sigmoid(alpha min(g, limit)) (clamp(u, -limit, limit) + shift).  As it
+// stands: SwiGLU, silu(g) u.
+struct Glu {
+  float alpha = 1.0f, limit = __builtin_inff(), shift = 0.0f;
+};
+
 // Arguments of one fused Linear launch:
-//   y = act(prologue(x) . W^T + bias) + residual
+//   y = act(prologue(x) . W^T + bias) * row_scale + residual
 // Output rows >= split1 / split2 are routed to y1 / y2 (fused-qkv rows going straight
 // into the K / V cache), offset by (pos[0] + m) * pos_stride floats.
 struct GemvArgs {
@@ -154,9 +160,11 @@ struct GemvArgs {
   // with fold_s: the Linear's own bias (may be null), so that a launch that prefers to normalise the staged
   // input itself can undo the folding (fold_s = null, bias = bias0)
   const float *bias0;
-  // rows 2r / 2r+1 are a (gate, up) pair: the launch writes silu(gate_r) * up_r to y[r] (rows/2 outputs)
-  // instead of the two products.  Needs a variant with at least two rows per wavefront.
+  const float *row_scale;  // a factor per output row (null = 1); launches that have one have a residual
+  // rows 2r / 2r+1 are a (gate, up) pair: the launch writes the gated unit of the two products to y[r] (rows/2 outputs)
+  // instead of the products.  Needs a variant with at least two rows per wavefront.
   int pair_swiglu;
+  Glu glu;  // the gated unit of pair_swiglu and of CTHIP_PRO_SWIGLU
   int stage_x;  // set by the launcher: the workgroup stages the input vector in LDS once
   float eps;
   float softcap;  // > 0: the stored value is softcap * tanh(value / softcap), before the argmax sees it
@@ -201,8 +209,8 @@ int gemv_rows_per_wave(int type, int64_t cols);
 // true when the single-row launch over a (rows, cols) matrix whose rows are gate / up rows in turn holds a row pair
 // per wavefront, so that SwiGLU can be its epilogue (layernorm: with a folded LayerNorm in front instead of an RMSNorm)
 bool gemv_pair_swiglu_ok(int type, int64_t rows, int64_t cols, bool layernorm = false);
-// out[i] = silu(in[2i]) * in[2i+1], i < n (gate / up columns interleaved)
-int launch_swiglu_pairs(float *out, const float *in, int64_t n);
+// out[i] = silu(in[2i]) * in[2i+1], i < n (gate / up columns interleaved), or the gated unit given
+int launch_swiglu_pairs(float *out, const float *in, int64_t n, Glu glu = Glu());
 // One query row over a long context: `ranges` workgroups per head share the keys (k_attn_cached, SPLIT).  part holds
 // H x ranges x (head_dim + 2) floats, count H zeroed ints (each launch leaves them zeroed again).
 struct AttnSplit {
@@ -247,21 +255,24 @@ struct GemmRoute {
   int ld[3];
 };
 // act == kActSwigluPairs: the weight rows are (gate_j, up_j) pairs and y (m, rows / 2) gets silu(gate_j) * up_j
-// (SwiGLU, external/llm/layers.lisp:53-64, in the epilogue of the gate|up launch); K is not split then.
+// (SwiGLU, external/llm/layers.lisp:53-64, in the epilogue of the gate|up launch), or the gated unit `glu`; K is not split then.
 constexpr int kActSwigluPairs = 64;
 // route: non-null = y is ignored, the columns go where the route says; K is not split then.
 int launch_linear_gemm(float *y, const WMat *w, const float *x, int m, const float *bias, const float *residual,
-                       int act, int precision, GemmDeferred *defer = nullptr, const GemmRoute *route = nullptr);
+                       int act, int precision, GemmDeferred *defer = nullptr, const GemmRoute *route = nullptr,
+                       const float *col_scale = nullptr, Glu glu = Glu());
 bool reduce_norm_supported(int n, int nparts);
-// C (m, n) = sum_z ws[z] + bias + residual for partial tiles handed over through GemmDeferred
-int launch_splitk_reduce(float *C, float *ws, int ksplit, int m, int n, const float *bias, const float *residual);
+// C (m, n) = (sum_z ws[z] + bias) * col_scale + residual for partial tiles handed over through GemmDeferred
+int launch_splitk_reduce(float *C, float *ws, int ksplit, int m, int n, const float *bias, const float *residual,
+                         const float *col_scale = nullptr);
 int launch_reduce_norm(float *y, float *xout, const float *parts, int nparts, int64_t part_stride, const float *bias,
-                       const float *resid, const float *g, const float *b, float eps, int64_t rows, int n, bool rms);
+                       const float *resid, const float *g, const float *b, float eps, int64_t rows, int n, bool rms,
+                       const float *col_scale = nullptr);
 // takes the device address of the static split-K scratch of cthip_matmul_noalloc (once per device, that device current)
 int matmul_scratch_init(int device);
 // gate|up rows (m, 2*cols) -> silu(gate)*up (m, cols), or a norm, as a launch of its own
 int launch_prologue(float *out, const float *x, int cols, int pro, const float *g, const float *b, float eps,
-                    int64_t x_stride, int m);
+                    int64_t x_stride, int m, Glu glu = Glu());
 // prefill: split fused qkv rows (S, D+2KD) into q (S,D) and cache rows start_pos.., rotating q and k when rope_base > 0
 int launch_qkv_split(float *q, float *kc, float *vc, const float *qkv, int S, int start_pos, int H, int Hkv, int Dh,
                      float rope_base);
@@ -379,6 +390,11 @@ __device__ __forceinline__ float ct_gelu(float x) {
 // cap * tanh(x / cap)
 __device__ __forceinline__ float softcap(float x, float cap) { return cap * ct_tanh(x / cap); }
 __device__ __forceinline__ float ct_silu(float x) { return x * ct_sigmoid(x); }
+__device__ __forceinline__ float gated_unit(float g, float u, const Glu &p) {
+  g = g > p.limit ? p.limit : g;
+  u = u > p.limit ? p.limit : u < -p.limit ? -p.limit : u;
+  return g * ct_sigmoid(p.alpha * g) * (u + p.shift);
+}
 __device__ __forceinline__ float apply_act(int act, float v) {
   switch (act) {
     case CTHIP_ACT_RELU: return fmaxf(v, 0.0f);

@@ -116,9 +116,9 @@ int dev_alloc(Decoder *d, void **p, size_t bytes);  // zero-filled, released wit
 int to_f32(Decoder *d, const std::string &key, int64_t want_n, float **out);
 int to_wmat(Decoder *d, const std::vector<std::string> &keys, int64_t want_rows, int64_t want_cols, WMat **out, bool interleave = false);
 int make_fold(Decoder *d, const WMat *w, const float *gamma, const float *beta, const float *bias, float **S, float **C);
-// X += W.in + bias over s rows, then XN = norm(X) with (g, b); g == nullptr: no norm follows
+// X += (W.in + bias) * col_scale over s rows, then XN = norm(X) with (g, b); g == nullptr: no norm follows
 int linear_residual_norm(float *XN, float *X, const WMat *w, const float *in, int s, int D, const float *bias, const float *g,
-                         const float *b, float eps, bool rms, int precision);
+                         const float *b, float eps, bool rms, int precision, const float *col_scale = nullptr);
 // decoder_mixed.hip
 void mixed_required(Decoder *d);
 int mixed_load(Decoder *d);              // the layers' matrices, states and caches out of the loaded tensors

@@ -806,17 +806,17 @@ static int queue_head(Decoder *d) {
 static const int kPrefillMin = 8;
 
 int linear_residual_norm(float *XN, float *X, const WMat *w, const float *in, int s, int D, const float *bias, const float *g,
-                         const float *b, float eps, bool rms, int precision) {
+                         const float *b, float eps, bool rms, int precision, const float *col_scale) {
   auto norm = [&]() { return rms ? cthip_rmsnorm(XN, X, g, eps, s, D) : cthip_layernorm(XN, X, g, b, eps, s, D); };
   GemmDeferred df;
   const bool fuse = g != nullptr && reduce_norm_supported(D, 1);
-  int r = launch_linear_gemm(X, w, in, s, bias, X, CTHIP_ACT_NONE, precision, fuse ? &df : nullptr);
+  int r = launch_linear_gemm(X, w, in, s, bias, X, CTHIP_ACT_NONE, precision, fuse ? &df : nullptr, nullptr, col_scale);
   if (r) return r;
   if (df.ws) {
     if (reduce_norm_supported(D, df.ksplit)) {
-      r = launch_reduce_norm(XN, X, df.ws, df.ksplit, (int64_t)s * D, bias, X, g, b, eps, s, D, rms);
+      r = launch_reduce_norm(XN, X, df.ws, df.ksplit, (int64_t)s * D, bias, X, g, b, eps, s, D, rms, col_scale);
     } else {  // too many shares of too wide a row to hold at once: reduce, then normalise
-      r = launch_splitk_reduce(X, df.ws, df.ksplit, s, D, bias, X);
+      r = launch_splitk_reduce(X, df.ws, df.ksplit, s, D, bias, X, col_scale);
       if (!r) r = norm();
     }
     const int r2 = cthip_free(df.ws);  // stream-ordered: reused only by later work on this stream

@@ -111,13 +111,13 @@ __device__ __forceinline__ void argmax_merge(float &v, int &i, float ov, int oi)
   }
 }
 
-// Epilogue shared by the GEMV kernels: bias, activation, residual, routing of fused-qkv rows.
+// Epilogue shared by the GEMV kernels: bias, activation, row factor, residual, routing of fused-qkv rows.
 __device__ __forceinline__ float gemv_store(const GemvArgs &a, int m, int row, float acc, int posv, float bias,
-                                            float resid) {
+                                            float resid, float scale) {
   float v = acc + bias;
   v = apply_act(a.act, v);
   if (a.softcap > 0.0f) v = softcap(v, a.softcap);
-  v += resid;
+  v = fmaf(v, scale, resid);
   float *dst;
   if (row < a.split1) {
     dst = a.y + (int64_t)m * a.y_stride + row;
@@ -158,7 +158,7 @@ __device__ __forceinline__ void coop_prologue(const GemvArgs &a, const float *__
     for (int i = tid; i < n4; i += nthr) {
       float4 v = ((const float4 *)x)[i];
       float4 u = ((const float4 *)(x + (a.up_off ? a.up_off : a.cols)))[i];
-      ((float4 *)xs)[i] = make_float4(ct_silu(v.x) * u.x, ct_silu(v.y) * u.y, ct_silu(v.z) * u.z, ct_silu(v.w) * u.w);
+      ((float4 *)xs)[i] = make_float4(gated_unit(v.x, u.x, a.glu), gated_unit(v.y, u.y, a.glu), gated_unit(v.z, u.z, a.glu), gated_unit(v.w, u.w, a.glu));
     }
     __syncthreads();
     return;
@@ -379,15 +379,16 @@ __device__ __forceinline__ void gemv_ring(const GemvArgs &a, float *xs_lds, floa
       }
     }
     // the epilogue operands of the row travel with its weights, in ONE request: the first three lanes of the
-    // row's group fetch bias, residual and fold term, and the group's first lane collects them with two lane
-    // shifts when it stores.  Lanes with nothing to fetch repeat a neighbour's address: a common dummy line
+    // row's group (four with a row factor) fetch bias, residual and fold term, and the group's first lane collects them
+    // with lane shifts when it stores.  Lanes with nothing to fetch repeat a neighbour's address: a common dummy line
     // would be re-fetched by every tile of every wavefront and its L2 channel would hold all of them up.
     if (EPI) {
       const float *pb = a.bias ? a.bias + row : nullptr;
       const float *pr = a.residual ? a.residual + (int64_t)m * a.y_stride + row : nullptr;
       const float *pf = a.fold_s ? a.fold_s + row : nullptr;
+      const float *ps = a.row_scale ? a.row_scale + row : nullptr;  // (never alone: there is a residual then)
       const float *any = pb ? pb : pr ? pr : pf;  // one of them exists, or the launcher takes the kernel without EPI
-      epi = *(l == 0 ? (pb ? pb : any) : l == 1 ? (pr ? pr : any) : l == 2 ? (pf ? pf : any) : any);
+      epi = *(l == 0 ? (pb ? pb : any) : l == 1 ? (pr ? pr : any) : l == 2 ? (pf ? pf : any) : l == 3 ? (ps ? ps : any) : any);
     }
   };
   uint4 wt[PD][KC];
@@ -430,7 +431,7 @@ __device__ __forceinline__ void gemv_ring(const GemvArgs &a, float *xs_lds, floa
     const float pivot = layernorm ? sv[0].x : 0.0f;  // this thread's first element (threads without one sum nothing)
     auto put = [&](int i, const float4 v, const float4 u) {
       if (swiglu) {
-        ((float4 *)xs_lds)[i] = make_float4(ct_silu(v.x) * u.x, ct_silu(v.y) * u.y, ct_silu(v.z) * u.z, ct_silu(v.w) * u.w);
+        ((float4 *)xs_lds)[i] = make_float4(gated_unit(v.x, u.x, a.glu), gated_unit(v.y, u.y, a.glu), gated_unit(v.z, u.z, a.glu), gated_unit(v.w, u.w, a.glu));
       } else if (folded || direct) {
         const float4 gm = a.norm_g ? u : make_float4(1.f, 1.f, 1.f, 1.f);
         const float d0 = v.x - pivot, d1 = v.y - pivot, d2 = v.z - pivot, d3 = v.w - pivot;
@@ -591,12 +592,13 @@ __device__ __forceinline__ void gemv_ring(const GemvArgs &a, float *xs_lds, floa
     const float bias = (EPI && a.bias) ? epi_t[p] : 0.0f;
     const float resid = (EPI && a.residual) ? dpp_f<0x101>(epi_t[p]) : 0.0f;  // row_shl:1
     const float fs = (EPI && a.fold_s) ? dpp_f<0x102>(epi_t[p]) : 0.0f;       // row_shl:2
+    const float sc = (EPI && a.row_scale) ? dpp_f<0x103>(epi_t[p]) : 1.0f;    // row_shl:3
     if (folded) acc = rstd * (acc - mu * fs);
     const int row = rq * RPW + g;
     if (PAIR1) {
       // SwiGLU across the (gate, up) row pair held by two neighbouring ring slots of this wavefront
       if (p & 1) {
-        if (l == 0 && row < a.rows) a.y[(int64_t)m * a.y_stride + (row >> 1)] = ct_silu(held_gate) * (acc + bias);
+        if (l == 0 && row < a.rows) a.y[(int64_t)m * a.y_stride + (row >> 1)] = gated_unit(held_gate, acc + bias, a.glu);
       } else {
         held_gate = acc + bias;
       }
@@ -604,9 +606,9 @@ __device__ __forceinline__ void gemv_ring(const GemvArgs &a, float *xs_lds, floa
       // SwiGLU across the (gate, up) row pair held by neighbouring lane groups
       const float mine = acc + bias;
       const float other = __shfl_xor(mine, G & 63, 64);
-      if (l == 0 && (g & 1) == 0 && row < a.rows) a.y[(int64_t)m * a.y_stride + (row >> 1)] = ct_silu(mine) * other;
+      if (l == 0 && (g & 1) == 0 && row < a.rows) a.y[(int64_t)m * a.y_stride + (row >> 1)] = gated_unit(mine, other, a.glu);
     } else if (l == 0 && row < a.rows) {
-      const float v = gemv_store(a, m, row, acc, posv, bias, resid);
+      const float v = gemv_store(a, m, row, acc, posv, bias, resid, sc);
       argmax_merge(best_v, best_i, v, row);
     }
   };
@@ -665,13 +667,14 @@ __global__ __launch_bounds__(256) void k_gemv(GemvArgs a) {
   // end of a row reads the zero block, an absent epilogue operand reads the zero block): a load behind a branch
   // leaves a copy of its result at the end of that branch, and the wavefront would wait there for the whole tile
   // before it has even requested its input vector -- two memory round trips in a launch that is nothing but latency.
-  auto load = [&](int rq, uint4 *w, unsigned *s, float &bias, float &resid, float &fs) {
+  auto load = [&](int rq, uint4 *w, unsigned *s, float &bias, float &resid, float &fs, float &sc) {
     int row = rq * RPW + g;
     row = row < a.rows ? row : a.rows - 1;
     const float *zf = (const float *)g_gemv_zeros;
     bias = *(a.bias ? a.bias + row : zf);
     resid = *(a.residual ? a.residual + (int64_t)m * a.y_stride + row : zf);
     fs = *(a.fold_s ? a.fold_s + row : zf);
+    sc = *(a.row_scale ? a.row_scale + row : zf);
 #pragma unroll
     for (int j = 0; j < KC; j++) {
       const int c = l + G * j;
@@ -695,11 +698,11 @@ __global__ __launch_bounds__(256) void k_gemv(GemvArgs a) {
   // (one 32-bit register per scale: 16-bit elements would be packed in pairs right behind their loads, and that
   // use would make the wavefront wait for the tile before it has requested anything else)
   unsigned st[PD][KC];
-  float bias_t[PD], resid_t[PD], fs_t[PD];
+  float bias_t[PD], resid_t[PD], fs_t[PD], sc_t[PD];
 #pragma unroll
   for (int p = 0; p < PD; p++) {
     const int rq = wave + p * total_waves;
-    load(rq < nrq ? rq : nrq - 1, wt[p], st[p], bias_t[p], resid_t[p], fs_t[p]);
+    load(rq < nrq ? rq : nrq - 1, wt[p], st[p], bias_t[p], resid_t[p], fs_t[p], sc_t[p]);
   }
 
   float xr[KC][XPC];
@@ -791,13 +794,13 @@ __global__ __launch_bounds__(256) void k_gemv(GemvArgs a) {
           // SwiGLU across the (gate, up) row pair held by neighbouring lane groups
           const float mine = acc + bias_t[p];
           const float other = __shfl_xor(mine, G & 63, 64);
-          if (l == 0 && (g & 1) == 0 && row < a.rows) a.y[(int64_t)m * a.y_stride + (row >> 1)] = ct_silu(mine) * other;
+          if (l == 0 && (g & 1) == 0 && row < a.rows) a.y[(int64_t)m * a.y_stride + (row >> 1)] = gated_unit(mine, other, a.glu);
         } else if (l == 0 && row < a.rows) {
-          const float v = gemv_store(a, m, row, acc, posv, bias_t[p], resid_t[p]);
+          const float v = gemv_store(a, m, row, acc, posv, bias_t[p], resid_t[p], a.row_scale ? sc_t[p] : 1.0f);
           argmax_merge(best_v, best_i, v, row);
         }
         const int nxt = rq + PD * total_waves;
-        if (nxt < nrq) load(nxt, wt[p], st[p], bias_t[p], resid_t[p], fs_t[p]);
+        if (nxt < nrq) load(nxt, wt[p], st[p], bias_t[p], resid_t[p], fs_t[p], sc_t[p]);
       }
     }
   }

@@ -70,12 +70,13 @@ void k_gemv_wide(GemvArgs a, int tpr) {
         if (RW > 1) st[p][RW - 1][k] = *(ok ? a.d + (int64_t)row1 * scales_per_row + sidx : (const unsigned short *)g_gemv_zeros);
       }
     }
-    // the rows' bias and residual travel with their tiles: lanes 0, 1 ask for row0's, lanes 2, 3 for row1's
-    const int er = (lane & 2) ? row1 : row0;
+    // the rows' bias, residual and factor travel with their tiles: lanes 0, 1, 2 ask for row0's, lanes 4, 5, 6 for row1's
+    const int er = (lane & 4) ? row1 : row0;
     const float *pb = a.bias ? a.bias + er : nullptr;
     const float *pr = a.residual ? a.residual + (int64_t)m * a.y_stride + er : nullptr;
     const float *any = pb ? pb : pr ? pr : (const float *)g_gemv_zeros;
-    epi_t[p] = *((lane & 1) ? (pr ? pr : any) : (pb ? pb : any));
+    const float *ps = a.row_scale ? a.row_scale + er : any;
+    epi_t[p] = *((lane & 2) ? ps : (lane & 1) ? (pr ? pr : any) : (pb ? pb : any));
     // advance; past the last tile the last one is requested again (and never consumed)
     if (rq_left > 1) {
       rq_left--;
@@ -108,7 +109,7 @@ void k_gemv_wide(GemvArgs a, int tpr) {
       if (i < n4) {
         const float4 v = vb[b], u = ub[b];
         float4 o = v;
-        if (swiglu) o = make_float4(ct_silu(v.x) * u.x, ct_silu(v.y) * u.y, ct_silu(v.z) * u.z, ct_silu(v.w) * u.w);
+        if (swiglu) o = make_float4(gated_unit(v.x, u.x, a.glu), gated_unit(v.y, u.y, a.glu), gated_unit(v.z, u.z, a.glu), gated_unit(v.w, u.w, a.glu));
         if (rms) {
           s2 = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, s2))));
           if (a.norm_g) o = make_float4(v.x * u.x, v.y * u.y, v.z * u.z, v.w * u.w);
@@ -167,12 +168,13 @@ void k_gemv_wide(GemvArgs a, int tpr) {
       const float s0 = wave_sum(acc0) * rstd, s1 = RW > 1 ? wave_sum(acc1) * rstd : 0.0f;
       const int row0 = RW * cs_pair;
       const float b0 = a.bias ? __shfl(row_epi, 0, 64) : 0.0f, r0 = a.residual ? __shfl(row_epi, 1, 64) : 0.0f;
-      const float b1 = a.bias ? __shfl(row_epi, 2, 64) : 0.0f, r1 = a.residual ? __shfl(row_epi, 3, 64) : 0.0f;
+      const float b1 = a.bias ? __shfl(row_epi, 4, 64) : 0.0f, r1 = a.residual ? __shfl(row_epi, 5, 64) : 0.0f;
+      const float f0 = a.row_scale ? __shfl(row_epi, 2, 64) : 1.0f, f1 = a.row_scale ? __shfl(row_epi, 6, 64) : 1.0f;
       if (RW > 1 && a.pair_swiglu) {  // the pair is a (gate, up) row pair: SwiGLU here, one output per pair
-        if (lane == 0) a.y[(int64_t)m * a.y_stride + (row0 >> 1)] = ct_silu(s0 + b0) * (s1 + b1);
+        if (lane == 0) a.y[(int64_t)m * a.y_stride + (row0 >> 1)] = gated_unit(s0 + b0, s1 + b1, a.glu);
       } else {
-        if (lane == 0) gemv_store(a, m, row0, s0, posv, b0, r0);
-        if (RW > 1 && lane == 1 && row0 + 1 < a.rows) gemv_store(a, m, row0 + 1, s1, posv, b1, r1);
+        if (lane == 0) gemv_store(a, m, row0, s0, posv, b0, r0, f0);
+        if (RW > 1 && lane == 1 && row0 + 1 < a.rows) gemv_store(a, m, row0 + 1, s1, posv, b1, r1, f1);
       }
       acc0 = acc1 = 0.0f;
       cs_grp = 0;

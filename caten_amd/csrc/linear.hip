@@ -243,7 +243,7 @@ __global__ __launch_bounds__(256) void k_gemv_generic(GemvArgs a) {
     acc = wave_sum(acc);
     if (lane == 0) {
       const float v = gemv_store(a, m, row, acc, posv, a.bias ? a.bias[row] : 0.0f,
-                                 a.residual ? a.residual[(int64_t)m * a.y_stride + row] : 0.0f);
+                                 a.residual ? a.residual[(int64_t)m * a.y_stride + row] : 0.0f, a.row_scale ? a.row_scale[row] : 1.0f);
       argmax_merge(best_v, best_i, v, row);
     }
   }
@@ -274,7 +274,7 @@ __global__ __launch_bounds__(256) void k_gemv_elements(GemvArgs a) {
     acc = wave_sum(acc);
     if (lane == 0) {
       const float v = gemv_store(a, m, row, acc, posv, a.bias ? a.bias[row] : 0.0f,
-                                 a.residual ? a.residual[(int64_t)m * a.y_stride + row] : 0.0f);
+                                 a.residual ? a.residual[(int64_t)m * a.y_stride + row] : 0.0f, a.row_scale ? a.row_scale[row] : 1.0f);
       argmax_merge(best_v, best_i, v, row);
     }
   }
@@ -284,7 +284,7 @@ __global__ __launch_bounds__(256) void k_gemv_elements(GemvArgs a) {
 // prologue as a kernel of its own, for the generic fallback: one block per input vector
 __global__ __launch_bounds__(256) void k_prologue(float *__restrict__ out, const float *__restrict__ x, int cols,
                                                   int pro, const float *__restrict__ g,
-                                                  const float *__restrict__ b, float eps, int64_t x_stride) {
+                                                  const float *__restrict__ b, float eps, int64_t x_stride, Glu glu) {
   __shared__ float red[4];
   const float *xi = x + (int64_t)blockIdx.x * x_stride;
   float *o = out + (int64_t)blockIdx.x * cols;
@@ -297,7 +297,7 @@ __global__ __launch_bounds__(256) void k_prologue(float *__restrict__ out, const
     return red[0] + red[1] + red[2] + red[3];
   };
   if (pro == CTHIP_PRO_SWIGLU) {
-    for (int i = tid; i < cols; i += 256) o[i] = ct_silu(xi[i]) * xi[cols + i];
+    for (int i = tid; i < cols; i += 256) o[i] = gated_unit(xi[i], xi[cols + i], glu);
     return;
   }
   float mean = 0.0f;
@@ -350,24 +350,24 @@ static const GemvVariant *pick_variant(int type, int cols) { return variant_of(g
 // silu(gate) * up of m rows laid out (gate[cols], up[cols]): element-wise, so a row is spread over as many workgroups
 // as it has blocks of 1024 elements (one workgroup per row took 35 us for the 28672 features of a 70B-shape FFN)
 __global__ __launch_bounds__(256) void k_swiglu_rows(float *__restrict__ out, const float *__restrict__ x, int cols,
-                                                     int64_t x_stride) {
+                                                     int64_t x_stride, Glu glu) {
   const float *xi = x + (int64_t)blockIdx.y * x_stride;
   float *o = out + (int64_t)blockIdx.y * cols;
   const int i0 = blockIdx.x * 1024 + threadIdx.x;
 #pragma unroll
   for (int k = 0; k < 4; k++) {
     const int i = i0 + 256 * k;
-    if (i < cols) o[i] = ct_silu(xi[i]) * xi[cols + i];
+    if (i < cols) o[i] = gated_unit(xi[i], xi[cols + i], glu);
   }
 }
 
 int launch_prologue(float *out, const float *x, int cols, int pro, const float *g, const float *b, float eps,
-                    int64_t x_stride, int m) {
+                    int64_t x_stride, int m, Glu glu) {
   if (m == 0) return 0;
   if (pro == CTHIP_PRO_SWIGLU)
-    hipLaunchKernelGGL(k_swiglu_rows, dim3((unsigned)((cols + 1023) / 1024), (unsigned)m), dim3(256), 0, state().stream, out, x, cols, x_stride);
+    hipLaunchKernelGGL(k_swiglu_rows, dim3((unsigned)((cols + 1023) / 1024), (unsigned)m), dim3(256), 0, state().stream, out, x, cols, x_stride, glu);
   else
-    hipLaunchKernelGGL(k_prologue, dim3(m), dim3(256), 0, state().stream, out, x, cols, pro, g, b, eps, x_stride);
+    hipLaunchKernelGGL(k_prologue, dim3(m), dim3(256), 0, state().stream, out, x, cols, pro, g, b, eps, x_stride, glu);
   CTHIP_LAUNCH_CHECK();
   return 0;
 }
@@ -413,17 +413,17 @@ int gemv_rows_per_wave(int type, int64_t cols) {
   return v ? 64 / v->G : 0;
 }
 
-__global__ __launch_bounds__(256) void k_swiglu_pairs(float *__restrict__ out, const float *__restrict__ in, int64_t n) {
+__global__ __launch_bounds__(256) void k_swiglu_pairs(float *__restrict__ out, const float *__restrict__ in, int64_t n, Glu glu) {
   for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
     const float2 v = ((const float2 *)in)[i];
-    out[i] = ct_silu(v.x) * v.y;
+    out[i] = gated_unit(v.x, v.y, glu);
   }
 }
-int launch_swiglu_pairs(float *out, const float *in, int64_t n) {
+int launch_swiglu_pairs(float *out, const float *in, int64_t n, Glu glu) {
   if (n <= 0) return 0;
   int64_t blocks = (n + 255) / 256;
   if (blocks > 8192) blocks = 8192;
-  hipLaunchKernelGGL(k_swiglu_pairs, dim3((unsigned)blocks), dim3(256), 0, state().stream, out, in, n);
+  hipLaunchKernelGGL(k_swiglu_pairs, dim3((unsigned)blocks), dim3(256), 0, state().stream, out, in, n, glu);
   CTHIP_LAUNCH_CHECK();
   return 0;
 }
@@ -496,6 +496,7 @@ int launch_gemv(const WMat *w, GemvArgs a, int m) {
   a.ld_chunks = a.ld_scales = a.up_off = 0;
   if (a.split1 <= 0) a.split1 = a.split2 = a.rows;
   if (a.am_val && m != 1) return fail(CTHIP_E_BAD_ARG, "gemv: the fused argmax needs m == 1");
+  if (a.row_scale && !a.residual) return fail(CTHIP_E_BAD_ARG, "gemv: a factor per row comes with a residual");
   const GemvVariant *v = pick_variant(w->type, a.cols);
   if (gemv_prefers_wide(v, w->type, a.rows) && gemv_wide_supported(w, a)) return launch_gemv_wide(w, a, m);
   if (a.pair_swiglu && (!v || (a.rows & 1) || a.am_val || a.residual || a.split1 != a.rows))
@@ -536,7 +537,7 @@ int launch_gemv(const WMat *w, GemvArgs a, int m) {
   if (a.pro != CTHIP_PRO_NONE) {
     int rc = alloc_scratch((void **)&tmp, sizeof(float) * (size_t)a.cols * m);  // fully written below
     if (rc) return rc;
-    rc = launch_prologue(tmp, a.x, a.cols, a.pro, a.norm_g, a.norm_b, a.eps, a.x_stride, m);
+    rc = launch_prologue(tmp, a.x, a.cols, a.pro, a.norm_g, a.norm_b, a.eps, a.x_stride, m, a.glu);
     if (rc) {
       cthip_free(tmp);
       return rc;

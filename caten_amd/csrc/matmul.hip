@@ -29,6 +29,7 @@ struct GemmArgs {
   int wtype;
   const float *bias;     // per output column, may be null
   const float *residual; // (M,N), may be null
+  const float *scale;    // per output column, between activation and residual; may be null
   int M, N, K;
   int act;
   // split-K: workgroup (tile, z) covers k in [z * kper, (z + 1) * kper) and writes
@@ -39,7 +40,8 @@ struct GemmArgs {
   // rm x rn tiles, one per XCD (workgroup i is dispatched to XCD i % 8), so that every L2 holds only
   // its region's rows of A and columns of B
   int tm, tn, rx, rm, rn;
-  int pairs;        // 1: columns (2j, 2j + 1) are (gate, up) and C (M, N / 2) gets silu(gate) * up
+  int pairs;        // 1: columns (2j, 2j + 1) are (gate, up) and C (M, N / 2) gets silu(gate) * up (or the gated unit glu)
+  Glu glu;
   int routed;       // 1: whole tiles go to route.dst[...] instead of C (see GemmRoute)
   GemmRoute route;
 };
@@ -152,7 +154,7 @@ __device__ __forceinline__ void store_tile(const GemmArgs &a, const float *Cs, i
         v[0] += bb.x, v[1] += bb.y, v[2] += bb.z, v[3] += bb.w;
       }
       *(float2 *)(a.C + (int64_t)row * (N >> 1) + (col >> 1)) =
-          make_float2(apply_act(CTHIP_ACT_SILU, v[0]) * v[1], apply_act(CTHIP_ACT_SILU, v[2]) * v[3]);
+          make_float2(gated_unit(v[0], v[1], a.glu), gated_unit(v[2], v[3], a.glu));
       continue;
     }
     if (vec) {
@@ -163,6 +165,10 @@ __device__ __forceinline__ void store_tile(const GemmArgs &a, const float *Cs, i
         }
 #pragma unroll
         for (int t = 0; t < 4; t++) v[t] = apply_act(a.act, v[t]);
+        if (a.scale) {
+          const float4 ss = *(const float4 *)(a.scale + col);
+          v[0] *= ss.x, v[1] *= ss.y, v[2] *= ss.z, v[3] *= ss.w;
+        }
         if (a.residual) {
           const float4 rr = *(const float4 *)(a.residual + (int64_t)row * N + col);
           v[0] += rr.x, v[1] += rr.y, v[2] += rr.z, v[3] += rr.w;
@@ -174,6 +180,7 @@ __device__ __forceinline__ void store_tile(const GemmArgs &a, const float *Cs, i
         float x = v[t];
         if (!plain) {
           x = apply_act(a.act, x + (a.bias ? a.bias[col + t] : 0.0f));
+          if (a.scale) x *= a.scale[col + t];
           if (a.residual) x += a.residual[(int64_t)row * N + col + t];
         }
         o[t] = x;
@@ -1079,7 +1086,7 @@ __global__ __launch_bounds__(768) void k_gemm_f32pc(GemmArgs a) {
   store_tile<BM, BN, 768>(a, Cs, m0, n0, tid);
 }
 
-// C = act(sum_z ws[z] + bias) + residual, z in ascending order (the result does not depend on timing)
+// C = act(sum_z ws[z] + bias) * scale + residual, z in ascending order (the result does not depend on timing)
 __global__ __launch_bounds__(256) void k_splitk_reduce(GemmArgs a) {
   const int64_t n = (int64_t)a.M * a.N;
   // Up to eight partials, bias and residual are requested together, none behind a branch (absent ones re-read
@@ -1088,6 +1095,7 @@ __global__ __launch_bounds__(256) void k_splitk_reduce(GemmArgs a) {
   for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
     const float bv = *(a.bias ? a.bias + i % a.N : a.ws + i);
     const float rv = *(a.residual ? a.residual + i : a.ws + i);
+    const float sv = *(a.scale ? a.scale + i % a.N : a.ws + i);
     float v = 0.0f;
     for (int zb = 0; zb < a.ksplit; zb += 8) {
       float t[8];
@@ -1099,6 +1107,7 @@ __global__ __launch_bounds__(256) void k_splitk_reduce(GemmArgs a) {
     }
     if (a.bias) v += bv;
     v = apply_act(a.act, v);
+    if (a.scale) v *= sv;
     if (a.residual) v += rv;
     a.C[i] = v;
   }
@@ -1272,8 +1281,8 @@ int launch_gemm(GemmArgs a, int bmode, int precision, float *static_ws, size_t s
   return 0;
 }
 
-// Linear over m rows with packed weights: y (m, rows) = act(x (m, cols) @ W^T + bias) + residual
-int launch_splitk_reduce(float *C, float *ws, int ksplit, int m, int n, const float *bias, const float *residual) {
+// Linear over m rows with packed weights: y (m, rows) = act(x (m, cols) @ W^T + bias) * col_scale + residual
+int launch_splitk_reduce(float *C, float *ws, int ksplit, int m, int n, const float *bias, const float *residual, const float *col_scale) {
   GemmArgs a = {};
   a.C = C;
   a.ws = ws;
@@ -1282,6 +1291,7 @@ int launch_splitk_reduce(float *C, float *ws, int ksplit, int m, int n, const fl
   a.N = n;
   a.bias = bias;
   a.residual = residual;
+  a.scale = col_scale;
   a.act = CTHIP_ACT_NONE;
   int64_t blocks = ((int64_t)m * n + 255) / 256;
   if (blocks > 4096) blocks = 4096;
@@ -1291,7 +1301,7 @@ int launch_splitk_reduce(float *C, float *ws, int ksplit, int m, int n, const fl
 }
 
 int launch_linear_gemm(float *y, const WMat *w, const float *x, int m, const float *bias, const float *residual,
-                       int act, int precision, GemmDeferred *defer, const GemmRoute *route) {
+                       int act, int precision, GemmDeferred *defer, const GemmRoute *route, const float *col_scale, Glu glu) {
   GemmArgs a = {};
   a.C = y;
   a.A = x;
@@ -1300,6 +1310,8 @@ int launch_linear_gemm(float *y, const WMat *w, const float *x, int m, const flo
   a.wtype = w->type;
   a.bias = bias;
   a.residual = residual;
+  a.scale = col_scale;
+  a.glu = glu;
   a.M = m;
   a.N = (int)w->rows;
   a.K = (int)w->cols;

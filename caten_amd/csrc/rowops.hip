@@ -128,7 +128,7 @@ __global__ __launch_bounds__(256) void k_rowop(RowArgs a) {
 // Split-K reduction, residual update and the following norm in one pass over the rows (prompt batches): a row-split
 // Linear whose reduction axis was shared among `nparts` workgroups per tile leaves raw partial tiles; the next thing
 // that happens to its output is the residual add and a LayerNorm / RMSNorm.  One wavefront per row:
-//   x = sum_z parts[z][row] (ascending z, as k_splitk_reduce adds them) + bias + resid   -> xout[row]
+//   x = (sum_z parts[z][row] (ascending z, as k_splitk_reduce adds them) + bias) * scale + resid   -> xout[row]
 //   y[row] = norm(x)                                                                    (arithmetic of k_rowop)
 struct ReduceNormArgs {
   float *y, *xout;
@@ -139,6 +139,7 @@ struct ReduceNormArgs {
   float eps;
   int64_t rows;
   int n;
+  const float *scale;  // per column, may be null
 };
 
 template <int MODE, int VPL, int NZ>
@@ -147,7 +148,7 @@ __global__ __launch_bounds__(256) void k_reduce_norm(ReduceNormArgs a) {
   const int64_t row = (int64_t)blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
   if (row >= a.rows) return;
   const int n = a.n, n4 = n >> 2;
-  float4 t[VPL][NZ], bs[VPL], rs[VPL], gm[VPL], bt[VPL];
+  float4 t[VPL][NZ], bs[VPL], rs[VPL], gm[VPL], bt[VPL], ss[VPL];
   bool ok[VPL];
   // every request first, none behind a branch: shares past nparts repeat share 0 and are dropped
 #pragma unroll
@@ -161,6 +162,7 @@ __global__ __launch_bounds__(256) void k_reduce_norm(ReduceNormArgs a) {
     rs[j] = ((const float4 *)((a.resid ? a.resid : a.parts) + row * n))[cc];
     gm[j] = ((const float4 *)(a.g ? a.g : a.parts))[cc];
     bt[j] = ((const float4 *)(a.b ? a.b : a.parts))[cc];
+    ss[j] = ((const float4 *)(a.scale ? a.scale : a.parts))[cc];
   }
   float v[VPL][4];
 #pragma unroll
@@ -170,6 +172,7 @@ __global__ __launch_bounds__(256) void k_reduce_norm(ReduceNormArgs a) {
     for (int z = 1; z < NZ; z++)
       if (z < a.nparts) x[0] += t[j][z].x, x[1] += t[j][z].y, x[2] += t[j][z].z, x[3] += t[j][z].w;
     if (a.bias) x[0] += bs[j].x, x[1] += bs[j].y, x[2] += bs[j].z, x[3] += bs[j].w;
+    if (a.scale) x[0] *= ss[j].x, x[1] *= ss[j].y, x[2] *= ss[j].z, x[3] *= ss[j].w;
     if (a.resid) x[0] += rs[j].x, x[1] += rs[j].y, x[2] += rs[j].z, x[3] += rs[j].w;
     if (ok[j]) ((float4 *)(a.xout + row * n))[lane + 64 * j] = make_float4(x[0], x[1], x[2], x[3]);
 #pragma unroll
@@ -215,7 +218,7 @@ __global__ __launch_bounds__(256) void k_reduce_norm_wide(ReduceNormArgs a) {
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
   const int64_t row = blockIdx.x;
   const int n = a.n, n4 = n >> 2;
-  float4 t[VPL][NZ], bs[VPL], rs[VPL], gm[VPL], bt[VPL];
+  float4 t[VPL][NZ], bs[VPL], rs[VPL], gm[VPL], bt[VPL], ss[VPL];
   bool ok[VPL];
   // every request first, none behind a branch: shares past nparts repeat share 0 and are dropped
 #pragma unroll
@@ -229,6 +232,7 @@ __global__ __launch_bounds__(256) void k_reduce_norm_wide(ReduceNormArgs a) {
     rs[j] = ((const float4 *)((a.resid ? a.resid : a.parts) + row * n))[cc];
     gm[j] = ((const float4 *)(a.g ? a.g : a.parts))[cc];
     bt[j] = ((const float4 *)(a.b ? a.b : a.parts))[cc];
+    ss[j] = ((const float4 *)(a.scale ? a.scale : a.parts))[cc];
   }
   float v[VPL][4];
 #pragma unroll
@@ -238,6 +242,7 @@ __global__ __launch_bounds__(256) void k_reduce_norm_wide(ReduceNormArgs a) {
     for (int z = 1; z < NZ; z++)
       if (z < a.nparts) x[0] += t[j][z].x, x[1] += t[j][z].y, x[2] += t[j][z].z, x[3] += t[j][z].w;
     if (a.bias) x[0] += bs[j].x, x[1] += bs[j].y, x[2] += bs[j].z, x[3] += bs[j].w;
+    if (a.scale) x[0] *= ss[j].x, x[1] *= ss[j].y, x[2] *= ss[j].z, x[3] *= ss[j].w;
     if (a.resid) x[0] += rs[j].x, x[1] += rs[j].y, x[2] += rs[j].z, x[3] += rs[j].w;
     if (ok[j]) ((float4 *)(a.xout + row * n))[tid + 256 * j] = make_float4(x[0], x[1], x[2], x[3]);
 #pragma unroll
@@ -283,10 +288,11 @@ __global__ __launch_bounds__(256) void k_reduce_norm_wide(ReduceNormArgs a) {
 bool reduce_norm_supported(int n, int nparts) { return reduce_norm_plan(n, nparts, 1).ok || reduce_norm_plan(n, nparts, 1 << 20).ok; }
 
 int launch_reduce_norm(float *y, float *xout, const float *parts, int nparts, int64_t part_stride, const float *bias,
-                       const float *resid, const float *g, const float *b, float eps, int64_t rows, int n, bool rms) {
+                       const float *resid, const float *g, const float *b, float eps, int64_t rows, int n, bool rms,
+                       const float *col_scale) {
   if (rows == 0 || n == 0) return 0;
   if (!reduce_norm_supported(n, nparts)) return fail(CTHIP_E_BAD_ARG, "reduce + norm: rows of %d with %d shares", n, nparts);
-  ReduceNormArgs a = {y, xout, parts, nparts, part_stride, bias, resid, g, b, eps, rows, n};
+  ReduceNormArgs a = {y, xout, parts, nparts, part_stride, bias, resid, g, b, eps, rows, n, col_scale};
   hipStream_t st = state().stream;
   const ReduceNormPlan pl = reduce_norm_plan(n, nparts, rows);
   if (pl.wide) {

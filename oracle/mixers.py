@@ -1,8 +1,8 @@
-"""Plain float64 restatement of the layers a mixed decoder is made of (gated delta rule, latent attention, gated
-feed-forward), one function per mechanism, token by token where the mechanism is a recurrence.  Test infrastructure:
-written from the equations, shares no code with the kernels, and is slow on purpose.
+"""Plain float64 restatement of the layers a mixed decoder is made of (gated delta rule, latent attention, sliding-window
+attention beside lightning attention, gated feed-forwards), one function per mechanism, token by token where the mechanism
+is a recurrence.  Test infrastructure: written from the equations, shares no code with the kernels, and is slow on purpose.
 
-A model is (config, tensors): the configuration dictionary of a Zuselix model directory and a dictionary
+A model is (config, tensors): the configuration dictionary of a Zuselix or Matalix model directory and a dictionary
 name -> float array.  Every function works on float64 NumPy arrays.
 """
 from __future__ import annotations
@@ -126,3 +126,102 @@ def zuselix(config, tensors, tokens):
     logits = layer_norm(x, t["final.norm"], eps) @ t["head"].T
     cap = config["logit_softcap"]
     return cap * np.tanh(logits / cap) if cap else logits, np.array(stream)
+
+
+# ---- Matalix ----
+def yarn(rot):
+    """rotation frequencies (dims / 2) and the factor of cosine and sine: slow rotations are stretched by `factor`, fast
+    ones are left, a linear ramp over the pair index lies between"""
+    dims, base, sc = rot["dims"], rot["base"], rot["scaling"]
+
+    def pair_that_turns(times):  # the (real-valued) pair that turns `times` times over the original context
+        return dims * np.log(sc["original"] / (2 * np.pi * times)) / (2 * np.log(base))
+    lo = max(np.floor(pair_that_turns(sc["fast"])), 0)
+    hi = min(np.ceil(pair_that_turns(sc["slow"])), dims - 1)
+    i = np.arange(dims // 2)
+    f = base ** (-2.0 * i / dims)
+    ramp = np.clip((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return f / sc["factor"] * ramp + f * (1.0 - ramp), 0.1 * np.log(sc["factor"]) + 1.0
+
+
+def rotate_half(x, positions, freqs, mscale):
+    """x (tokens, heads, dim): entries i and i + n of a head are a pair (n = len(freqs)), entries from 2 n on stay"""
+    n = len(freqs)
+    a = np.asarray(positions, np.float64)[:, None, None] * freqs
+    c, s = np.cos(a) * mscale, np.sin(a) * mscale
+    u, v = x[..., :n], x[..., n:2 * n]
+    return np.concatenate([u * c - v * s, v * c + u * s, x[..., 2 * n:]], -1)
+
+
+def window_attention(h, m, w, eps):
+    """grouped-query attention over the last mask.size positions; the softmax has a sink of score 0"""
+    T, H, G, dk, dv = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    freqs, mscale = yarn(m["rot"])
+    q = rms_norm(h @ w("q").T + w("q.b"), w("q.norm"), eps).reshape(T, H, dk)
+    k = rms_norm(h @ w("k").T + w("k.b"), w("k.norm"), eps).reshape(T, G, dk)
+    v = (h @ w("v").T + w("v.b")).reshape(T, G, dv)
+    q, k = rotate_half(q, range(T), freqs, mscale), rotate_half(k, range(T), freqs, mscale)
+    back = np.arange(T)[:, None] - np.arange(T)[None, :]
+    hidden = np.where((back >= 0) & (back < m["mask"]["size"]), 0.0, -np.inf)
+    o = np.zeros((T, H, dv))
+    for n in range(H):
+        g = n // (H // G)
+        o[:, n] = sink_softmax(q[:, n] @ k[:, g].T * m["scale"] + hidden, 0.0) @ v[:, g]
+    return (o.reshape(T, -1) * sigmoid(h @ w("g").T)) @ w("o").T
+
+
+def lightning_recurrence(q, k, v, decay):
+    """one head: q, k (tokens, dim), v (tokens, vdim); returns (o, final state)"""
+    S = np.zeros((k.shape[1], v.shape[1]))
+    o = np.zeros_like(v)
+    for t in range(len(q)):
+        S = decay * S + np.outer(k[t], v[t])
+        o[t] = S.T @ q[t]
+    return o, S
+
+
+def lightning_attention(h, m, w, eps):
+    T, H, dk, dv = h.shape[0], m["heads"], m["dim"], m["vdim"]
+    q, k = silu(h @ w("q").T).reshape(T, H, dk), silu(h @ w("k").T).reshape(T, H, dk)
+    v = silu(h @ w("v").T).reshape(T, H, dv)
+    o = np.zeros((T, H, dv))
+    for n in range(H):
+        o[:, n], _ = lightning_recurrence(q[:, n], k[:, n], v[:, n], m["decay"][n])
+    return (rms_norm(o.reshape(T, -1), w("norm"), eps) * sigmoid(h @ w("g").T)) @ w("o").T
+
+
+def parallel_mixer(h, m, w, eps):
+    return (m["left_scale"] * window_attention(h, m["left"], lambda n: w("left." + n), eps)
+            + m["right_scale"] * lightning_attention(h, m["right"], lambda n: w("right." + n), eps))
+
+
+def clamped_mlp(h, limit, w):
+    g = np.minimum(h @ w("gate").T, limit)
+    u = np.clip(h @ w("up").T, -limit, limit)
+    return (g * sigmoid(1.702 * g) * (u + 1.0)) @ w("down").T
+
+
+def matalix(config, tensors, tokens):
+    """-> (logits (tokens, vocab), residual stream after every layer run (layer runs, tokens, width))"""
+    t = {k: np.asarray(v, np.float64) for k, v in tensors.items()}
+    eps, loop = config["norm"]["eps"], config.get("loop") or {"start": 0, "stop": 0, "times": 1}
+    x0 = x = t["embed"][np.asarray(tokens)]
+    stream = []
+
+    def run(i, x):
+        layer, p = config["layers"][i], f"l{i}."
+        x = x + t[p + "ls1"] * parallel_mixer(rms_norm(x, 1.0 + t[p + "norm1"], eps), layer["mixer"], lambda n: t[p + "mix." + n], eps)
+        if layer["mlp"] is not None:
+            x = x + t[p + "ls2"] * clamped_mlp(rms_norm(x, 1.0 + t[p + "norm2"], eps), layer["mlp"]["limit"], lambda n: t[p + "mlp." + n])
+        stream.append(x)
+        return x
+    for i in range(loop["start"]):
+        x = run(i, x)
+    for p in range(loop["times"]):
+        if p:
+            x = x + x0
+        for i in range(loop["start"], loop["stop"]):
+            x = run(i, x)
+    for i in range(loop["stop"], len(config["layers"])):
+        x = run(i, x)
+    return rms_norm(x, 1.0 + t["final.norm"], eps) @ t["embed"].T, np.array(stream)
