@@ -18,7 +18,8 @@ GGML_TYPE = {"f32": F32, "f16": F16, "q4_0": Q4_0, "q8_0": Q8_0, "bf16": BF16}
 PRO_NONE, PRO_LAYERNORM, PRO_RMSNORM, PRO_SWIGLU = 0, 1, 2, 3
 ACT_NONE, ACT_RELU, ACT_GELU, ACT_SILU, ACT_SIGMOID, ACT_TANH = 0, 1, 2, 3, 4, 5
 ARCH_GPT2, ARCH_LLAMA, ARCH_MIXED = 0, 1, 2
-MIXER_DELTA, MIXER_LATENT = 0, 1
+MIXER_DELTA, MIXER_LATENT, MIXER_WINDOW, MIXER_LIGHTNING = 0, 1, 2, 3
+SINK_NONE, SINK_TENSOR, SINK_ZERO = 0, 1, 2
 
 
 class HipError(RuntimeError):
@@ -35,15 +36,24 @@ class DecoderConfig(C.Structure):
                 ("eps", C.c_float), ("rope_base", C.c_float)]
 
 
-class LayerSpec(C.Structure):
+class MixerSpec(C.Structure):
     _fields_ = [("mixer", C.c_int), ("heads", C.c_int), ("kv_heads", C.c_int), ("dim", C.c_int), ("vdim", C.c_int),
                 ("conv", C.c_int), ("kv_rank", C.c_int), ("scale", C.c_float), ("sink", C.c_int), ("gate", C.c_int),
-                ("ffn", C.c_int)]
+                ("window", C.c_int), ("bias", C.c_int), ("qk_norm", C.c_int), ("rot_dims", C.c_int), ("rot_base", C.c_double),
+                ("rot_factor", C.c_double), ("rot_original", C.c_double), ("rot_fast", C.c_double), ("rot_slow", C.c_double),
+                ("decay", C.POINTER(C.c_double)), ("out_scale", C.c_float)]
+
+
+class LayerSpec(C.Structure):
+    _fields_ = [("n_mixers", C.c_int), ("mixers", MixerSpec * 2), ("ffn", C.c_int), ("glu_alpha", C.c_float),
+                ("glu_limit", C.c_float), ("glu_shift", C.c_float), ("layer_scale", C.c_int)]
 
 
 class MixedConfig(C.Structure):
     _fields_ = [("n_layers", C.c_int), ("dim", C.c_int), ("vocab", C.c_int), ("max_seq", C.c_int), ("norm", C.c_int),
-                ("eps", C.c_float), ("position_base", C.c_float), ("logit_softcap", C.c_float), ("precision", C.c_int)]
+                ("eps", C.c_float), ("position_base", C.c_float), ("logit_softcap", C.c_float), ("precision", C.c_int),
+                ("norm_plus_one", C.c_int), ("tied_head", C.c_int), ("loop_start", C.c_int), ("loop_stop", C.c_int),
+                ("loop_times", C.c_int)]
 
 
 _vp, _vpp = C.c_void_p, C.POINTER(C.c_void_p)

@@ -6,7 +6,7 @@
 
 namespace cthip {
 
-// EXT: head sizes below the compiled ones (multiples of 4), a softmax sink, a gated output
+// EXT: head sizes below the compiled ones (multiples of 4), a softmax sink, a gated output, a sliding window
 static __device__ __align__(16) float g_attn_zeros[4];
 template <bool EXT>
 __device__ __forceinline__ float4 attn_piece(const float *p, int d, int n) {  // four floats at p + d, zeros past n
@@ -47,6 +47,9 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma(AttnRowsArgs a) {
   const int Tq = start_pos + qrow + 1;    // keys this lane's query sees
   const int Tmax = start_pos + min(i0 + 32, S);
   const int ntiles = (Tmax + 31) / 32;
+  // a window: keys from Tq - window on, tiles from the first row's first key on
+  const int Tlo = EXT && a.window > 0 ? Tq - a.window : 0;
+  const int tile0 = EXT && a.window > 0 ? max(start_pos + i0 + 1 - a.window, 0) >> 5 : 0;
   const float scale = a.scale;
   // the key tile of a pass is requested one pass ahead, its values at the start of the pass: both are in
   // registers by the time the matrix cores need them
@@ -59,7 +62,7 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma(AttnRowsArgs a) {
       kreg[u] = attn_piece<EXT>(kh + (int64_t)kr * a.ldk, 4 * d4, dk);
     }
   };
-  if (wv < ntiles) load_k(wv);
+  if (tile0 + wv < ntiles) load_k(tile0 + wv);
   // The block's 32 query rows go through LDS (the memory of the key tiles, before they are written): whole
   // rows in 16-byte pieces, one request per cache line and block.  (Every wavefront fetching its own operand
   // registers straight from memory asked for each line 128 times: 4 us of a 512-token launch.)
@@ -85,7 +88,7 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma(AttnRowsArgs a) {
 #pragma unroll
     for (int r = 0; r < 16; r++) o[b][r] = 0.0f;
 
-  for (int t = wv; t < ntiles; t += NW) {
+  for (int t = tile0 + wv; t < ntiles; t += NW) {
     const int kb = t * 32;
     // the key tile, transposed into LDS
 #pragma unroll
@@ -117,7 +120,7 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma(AttnRowsArgs a) {
 #pragma unroll
     for (int r = 0; r < 16; r++) {
       const int key = kb + 8 * (r >> 2) + 4 * half + (r & 3);
-      const float sc = (key < Tq) ? sacc[r] * scale : -INFINITY;
+      const float sc = (key < Tq && (!EXT || key >= Tlo)) ? sacc[r] * scale : -INFINITY;
       sacc[r] = sc;
       tmax = fmaxf(tmax, sc);
     }
@@ -154,7 +157,7 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma(AttnRowsArgs a) {
   __syncthreads();
   float M = Cm[0][lane];
 #pragma unroll
-  for (int w = 1; w < NW; w++) M = fmaxf(M, Cm[w][lane]);  // finite: the wavefront holding key 0 saw it
+  for (int w = 1; w < NW; w++) M = fmaxf(M, Cm[w][lane]);  // finite: every row sees its own key
   float e[NW], L = 0.0f;
 #pragma unroll
   for (int w = 0; w < NW; w++) {
@@ -182,6 +185,7 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma(AttnRowsArgs a) {
       const int dd = 32 * b + 8 * (r >> 2) + 4 * half + (r & 3);
       if (EXT && dd >= dv) continue;
       v *= inv;
+      if (EXT) v *= a.out_scale;
       if (grow) v *= ct_sigmoid(grow[dd]);
       orow[dd] = v;
     }
@@ -241,6 +245,9 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma_bf(AttnRowsArgs a) {
   const int Tq = start_pos + qrow + 1;    // keys this lane's query sees
   const int Tmax = start_pos + min(i0 + 32, S);
   const int ntiles = (Tmax + 31) / 32;
+  // a window: keys from Tq - window on, tiles from the first row's first key on
+  const int Tlo = EXT && a.window > 0 ? Tq - a.window : 0;
+  const int tile0 = EXT && a.window > 0 ? max(start_pos + i0 + 1 - a.window, 0) >> 5 : 0;
   const float scale = a.scale;
   // the key tile of a pass is requested one pass ahead, its values at the start of the pass
   float4 kreg[DK / 8];
@@ -252,7 +259,7 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma_bf(AttnRowsArgs a) {
       kreg[u] = attn_piece<EXT>(kh + (int64_t)kr * a.ldk, 4 * d4, dk);
     }
   };
-  if (wv < ntiles) load_k(wv);
+  if (tile0 + wv < ntiles) load_k(tile0 + wv);
   // the block's 32 query rows through LDS (the memory of the key tiles, before they are written), see k_attn_mfma
   constexpr int QP = DK + 4;
   static_assert(32 * QP * 4 <= sizeof(W), "the query rows fit the key tile memory");
@@ -277,7 +284,7 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma_bf(AttnRowsArgs a) {
 #pragma unroll
     for (int r = 0; r < 16; r++) o[b][r] = 0.0f;
 
-  for (int t = wv; t < ntiles; t += NW) {
+  for (int t = tile0 + wv; t < ntiles; t += NW) {
     const int kb = t * 32;
     // the key tile, split, into LDS
 #pragma unroll
@@ -316,7 +323,7 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma_bf(AttnRowsArgs a) {
 #pragma unroll
     for (int r = 0; r < 16; r++) {
       const int key = kb + 8 * (r >> 2) + 4 * half + (r & 3);
-      const float sc = (key < Tq) ? sacc[r] * scale : -INFINITY;
+      const float sc = (key < Tq && (!EXT || key >= Tlo)) ? sacc[r] * scale : -INFINITY;
       sacc[r] = sc;
       tmax = fmaxf(tmax, sc);
     }
@@ -362,7 +369,7 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma_bf(AttnRowsArgs a) {
   __syncthreads();
   float M = Cm[0][lane];
 #pragma unroll
-  for (int w = 1; w < NW; w++) M = fmaxf(M, Cm[w][lane]);  // finite: the wavefront holding key 0 saw it
+  for (int w = 1; w < NW; w++) M = fmaxf(M, Cm[w][lane]);  // finite: every row sees its own key
   float e[NW], L = 0.0f;
 #pragma unroll
   for (int w = 0; w < NW; w++) {
@@ -389,6 +396,7 @@ __global__ __launch_bounds__(64 * NW) void k_attn_mfma_bf(AttnRowsArgs a) {
       const int dd = 32 * b + 8 * (r >> 2) + 4 * half + (r & 3);
       if (EXT && dd >= dv) continue;
       v *= inv;
+      if (EXT) v *= a.out_scale;
       if (grow) v *= ct_sigmoid(grow[dd]);
       orow[dd] = v;
     }

@@ -39,16 +39,38 @@ struct Layer {
   void *proj_hq = nullptr, *proj_hd = nullptr, *fc2_sq = nullptr, *fc2_sd = nullptr;
 };
 
-// one layer of a mixed decoder (decoder_mixed.hip)
+// one mixer of a layer (decoder_mixed.hip): its rows of the layer's projection matrix start at row0, its output's columns
+// of the output matrix at col0
+struct MixedBranch {
+  cthip_mixer_spec sp;
+  std::string prefix;  // of its tensors' keys, behind "l<i>."
+  int64_t row0 = 0, col0 = 0;
+  WMat *absorb = nullptr, *kv_up = nullptr;  // latent: W_uk transposed per head; W_uk over W_uv
+  std::vector<double> decay;                 // lightning
+  // (everything but the projection rows and what a layer run keeps of the sequence)
+  DeltaArgs delta = {};
+  LatentArgs latent = {};
+  WindowArgs window = {};
+  LightningArgs lightning = {};
+};
+// one layer of a mixed decoder
 struct MixedLayer {
   cthip_layer_spec sp;
+  std::vector<MixedBranch> branches;
   float *norm1 = nullptr, *norm2 = nullptr;
   WMat *in = nullptr, *out = nullptr, *gate_up = nullptr, *down = nullptr;
+  float *bias = nullptr;                   // of `in`, where a projection has one
   float *in_s = nullptr, *fc_s = nullptr;  // LayerNorm folded through `in` / `gate_up`
-  bool fc_pairs = false;                   // gate / up rows interleaved, SwiGLU in that launch's epilogue
-  WMat *absorb = nullptr, *kv_up = nullptr;  // latent: W_uk transposed per head; W_uk over W_uv
-  DeltaArgs delta = {};    // (everything but the projection rows)
-  LatentArgs latent = {};
+  float *ls1 = nullptr, *ls2 = nullptr;    // factors of the mixer's and the feed-forward's results
+  bool fc_pairs = false;                   // gate / up rows interleaved, the gated unit in that launch's epilogue
+  Glu glu;
+  int64_t nbytes = 0;  // weights and vectors a run reads
+};
+// one run of a layer: looped layers run several times per token, each time with what that run has kept
+struct MixedRun {
+  int layer;
+  bool add_embedding;      // in front of it the embedding is added to the residual stream
+  float *keep[2][2] = {};  // per branch: delta ring, S; latent cache; window K, V; lightning S
 };
 
 struct Decoder {
@@ -59,7 +81,9 @@ struct Decoder {
   std::vector<Layer> layers;
   cthip_mixed_config mcfg = {};  // arch MIXED
   std::vector<MixedLayer> mixed;
+  std::vector<MixedRun> runs;
   LatentWork latent_work = {};
+  ParallelWork parallel_work = {};
   float *wte = nullptr, *wpe = nullptr, *lnf_g = nullptr, *lnf_b = nullptr;
   WMat *lm_head = nullptr;
   float *lm_s = nullptr, *lm_c = nullptr;  // ln_f folded through lm_head
@@ -124,7 +148,7 @@ void mixed_required(Decoder *d);
 int mixed_load(Decoder *d);              // the layers' matrices, states and caches out of the loaded tensors
 void mixed_release(Decoder *d);
 int mixed_queue_layers(Decoder *d);      // one decode step's layers, d->x in place
-int mixed_prefill(Decoder *d, float *X, float *XN, int s, int n);  // s rows at positions n .., X in place
+int mixed_prefill(Decoder *d, float *X, float *XN, const int *ids, int s, int n);  // s rows at positions n .., X in place
 int mixed_launches(const Decoder *d);    // the most launches any layer runs in a decode step
 int64_t mixed_state_bytes(const Decoder *d, int t);  // cache and state bytes of a step at position t
 int mixed_peek(Decoder *d, const char *what, void **ptr, int64_t *n_floats);  // 1 = not one of its buffers

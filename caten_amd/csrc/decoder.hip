@@ -908,7 +908,7 @@ static int prefill(Decoder *d, const int *ids, int s, int n, const int *rows, in
   }
   TRY(launch_embedding(X, d->wte, nullptr, ids_dev, s, V, D, d->wpe, d->tokpos + 1, c.max_seq));
   if (mixed) {
-    TRY(mixed_prefill(d, X, XN, s, n));
+    TRY(mixed_prefill(d, X, XN, ids_dev, s, n));
   } else {
     // A row-split Linear (attention projection, second MLP Linear) whose reduction axis was shared among several
     // workgroups per tile leaves partial tiles; what follows it is the residual add and the next norm, so one pass
@@ -1045,17 +1045,33 @@ int cthip_decoder_create_mixed(void **dec, const cthip_mixed_config *cfg, const 
   CTHIP_ARG(c.norm == CTHIP_PRO_LAYERNORM || c.norm == CTHIP_PRO_RMSNORM);
   CTHIP_ARG(c.precision >= -1 && c.precision <= GEMM_BF16X6);
   CTHIP_ARG(c.logit_softcap >= 0.0f && c.position_base >= 0.0f);
+  if (c.loop_times > 1) CTHIP_ARG(c.loop_start >= 0 && c.loop_start < c.loop_stop && c.loop_stop <= c.n_layers);
   for (int l = 0; l < c.n_layers; l++) {
-    const cthip_layer_spec &s = layers[l];
-    CTHIP_ARG(s.mixer == CTHIP_MIXER_DELTA || s.mixer == CTHIP_MIXER_LATENT);
-    CTHIP_ARG(s.heads > 0 && s.dim > 0 && s.vdim > 0 && s.ffn >= 0);
-    if (s.dim > 256 || s.vdim > 256)
-      return fail(CTHIP_E_UNSUPPORTED, "cthip_decoder_create_mixed: layer %d: heads of %d / %d (at most 256)", l, s.dim, s.vdim);
-    if (s.mixer == CTHIP_MIXER_DELTA) {
-      CTHIP_ARG(s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.conv > 0);
-    } else {
-      CTHIP_ARG(s.kv_rank > 0);
-      if (s.kv_rank > 1024) return fail(CTHIP_E_UNSUPPORTED, "cthip_decoder_create_mixed: layer %d: a latent of %d (at most 1024)", l, s.kv_rank);
+    const cthip_layer_spec &y = layers[l];
+    CTHIP_ARG(y.n_mixers == 1 || y.n_mixers == 2);
+    CTHIP_ARG(y.ffn >= 0 && y.glu_limit >= 0.0f);
+    for (int b = 0; b < y.n_mixers; b++) {
+      const cthip_mixer_spec &s = y.mixers[b];
+      CTHIP_ARG(s.mixer >= CTHIP_MIXER_DELTA && s.mixer <= CTHIP_MIXER_LIGHTNING);
+      CTHIP_ARG(s.heads > 0 && s.dim > 0 && s.vdim > 0);
+      if (s.dim > 256 || s.vdim > 256)
+        return fail(CTHIP_E_UNSUPPORTED, "cthip_decoder_create_mixed: layer %d: heads of %d / %d (at most 256)", l, s.dim, s.vdim);
+      if (s.mixer == CTHIP_MIXER_DELTA) {
+        CTHIP_ARG(s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.conv > 0);
+      } else if (s.mixer == CTHIP_MIXER_LATENT) {
+        CTHIP_ARG(s.kv_rank > 0);
+        CTHIP_ARG(s.sink >= 0 && s.sink <= CTHIP_SINK_TENSOR);
+        if (s.kv_rank > 1024) return fail(CTHIP_E_UNSUPPORTED, "cthip_decoder_create_mixed: layer %d: a latent of %d (at most 1024)", l, s.kv_rank);
+      } else if (s.mixer == CTHIP_MIXER_WINDOW) {
+        CTHIP_ARG(s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.window > 0);
+        CTHIP_ARG(s.sink >= 0 && s.sink <= CTHIP_SINK_ZERO);
+        CTHIP_ARG(s.rot_dims >= 0 && s.rot_dims % 2 == 0 && s.rot_dims <= s.dim && (s.rot_dims == 0 || s.rot_base > 0.0));
+      } else {
+        CTHIP_ARG(s.decay != nullptr);
+        for (int h = 0; h < s.heads; h++) CTHIP_ARG(s.decay[h] >= 0.0 && s.decay[h] <= 1.0);
+      }
+      if (y.n_mixers == 2 && s.mixer != CTHIP_MIXER_WINDOW && s.mixer != CTHIP_MIXER_LIGHTNING)
+        return fail(CTHIP_E_UNSUPPORTED, "cthip_decoder_create_mixed: layer %d: mixers of kind %d do not stand beside another", l, s.mixer);
     }
   }
   Decoder *d = new Decoder();
@@ -1069,7 +1085,26 @@ int cthip_decoder_create_mixed(void **dec, const cthip_mixed_config *cfg, const 
   d->cfg.max_seq = c.max_seq;
   d->cfg.eps = c.eps;
   d->mixed.resize(c.n_layers);
-  for (int l = 0; l < c.n_layers; l++) d->mixed[l].sp = layers[l];
+  for (int l = 0; l < c.n_layers; l++) {
+    MixedLayer &L = d->mixed[l];
+    L.sp = layers[l];
+    L.glu.alpha = L.sp.glu_alpha, L.glu.limit = L.sp.glu_limit, L.glu.shift = L.sp.glu_shift;
+    for (int b = 0; b < L.sp.n_mixers; b++) {
+      MixedBranch br;
+      br.sp = L.sp.mixers[b];
+      br.prefix = L.sp.n_mixers == 1 ? "mix." : b == 0 ? "mix.left." : "mix.right.";
+      if (br.sp.mixer == CTHIP_MIXER_LIGHTNING) br.decay.assign(br.sp.decay, br.sp.decay + br.sp.heads);
+      br.sp.decay = nullptr;  // (the caller's)
+      L.branches.push_back(br);
+    }
+  }
+  const int times = c.loop_times > 1 ? c.loop_times : 1, start = times > 1 ? c.loop_start : 0, stop = times > 1 ? c.loop_stop : 0;
+  for (int l = 0; l < c.n_layers; l++) {
+    if (l == start)
+      for (int pass = 1; pass < times; pass++)
+        for (int i = start; i < stop; i++) d->runs.push_back({i, pass > 1 && i == start});
+    d->runs.push_back({l, times > 1 && l == start});  // (the last pass of a looped layer)
+  }
   build_required(d);
   *dec = d;
   return 0;

@@ -1,5 +1,6 @@
-// The token mixers of decoders whose layers are listed one by one: the gated delta rule (delta.hip) and attention over
-// a cached latent vector (latent.hip).  Head sizes are padded to multiples of 16 in memory (zero rows and columns of
+// The token mixers of decoders whose layers are listed one by one: the gated delta rule (delta.hip), attention over
+// a cached latent vector (latent.hip), attention over a sliding window and lightning attention (window.hip, lightning.hip;
+// parallel.hip runs a decode step of the two side by side).  Head sizes are padded to multiples of 16 in memory (zero rows and columns of
 // the weights), so every row of a head is whole 16-byte pieces; the true sizes matter only where a mean is taken.
 #pragma once
 #include "common.h"
@@ -58,6 +59,60 @@ int launch_latent_step(const LatentArgs &a, const LatentWork &w, float *out, con
 // appends the latents of s tokens at rows n ..
 int launch_latent_append(const LatentArgs &a, int s, int n);
 
+// ---- attention over a sliding window ----
+// A projection row holds [q: H x DK | k: G x DK | v: G x DV | g: H x DV, where the output is gated].  Keys and values of
+// the last `rows` positions are kept in rings: position i in row i mod rows.
+struct WindowArgs {
+  const float *p;
+  int64_t ldp;
+  int H, G, DK, DV, dk, dv;
+  int window, rows;        // rows = min(window, longest sequence)
+  float eps, scale, out_scale;
+  const float *qnorm, *knorm;  // [H x DK], [G x DK], zeros in the padding; null = no norm
+  const float2 *rope;      // [position][half]: cosine and sine; null = no rotation
+  int half;                // entries i and i + half of a head are a pair, i < half
+  const float *sink;       // [H] logits of the extra softmax term; null = none
+  int gated;
+  float *K, *V;            // [rows][G x DK], [rows][G x DV]
+};
+// queries and keys of s rows normalised and rotated, queries in place; keys and values of the visible earlier rows and of
+// these -> kbuf (prev + s, G x DK), vbuf (prev + s, G x DV), prev = window_prev(a, n)
+int window_prev(const WindowArgs &a, int n);
+int launch_window_prepare(const WindowArgs &a, float *p, float *kbuf, float *vbuf, int s, int n);
+// the last rows of kbuf / vbuf into the rings
+int launch_window_keep(const WindowArgs &a, const float *kbuf, const float *vbuf, int s, int n);
+
+// ---- lightning attention ----
+// A projection row holds [q: H x DK | k: H x DK | v: H x DV | g: H x DV].
+struct LightningArgs {
+  const float *p;
+  int64_t ldp;
+  int H, DK, DV, dk, dv;
+  const float *decay;      // [3][H]: the decay less 1, its logarithm to base 2, the decay itself
+  const float *norm;       // [H x DV], zeros in the padding
+  float eps, out_scale;
+  float *S;                // [H][DV][DK], fp32
+};
+// s tokens at positions n .. n + s - 1 -> out rows ldo floats apart; p: the projection rows, q, k and v of which pass silu
+// in place; scratch: lightning_scratch_floats() floats
+size_t lightning_scratch_floats(const LightningArgs &a, int s);
+int launch_lightning_rows(const LightningArgs &a, float *p, float *out, int64_t ldo, int s, int n, float *scratch);
+
+// ---- a decode step of either, or of both side by side in one launch ----
+struct ParallelWork {
+  float *part;   // window: every key range's unnormalised sums, maximum and denominator
+  int *count;    // tickets: one for the lightning heads, then window_tickets() of them; zeroed (each launch leaves them zeroed again)
+  float *raw;    // lightning: H x DV outputs before the norm, then a sum of squares per workgroup
+};
+constexpr int kWindowMaxRanges = 16;
+int window_tickets(const WindowArgs &a);
+size_t window_part_floats(const WindowArgs &a);
+size_t lightning_raw_floats(const LightningArgs &a);
+// w -> wout (H x DV), l -> lout (H x DV); either may be null.  The token at position tokpos[1]; once ctrl[1] is set (the
+// sequence has ended) the recurrent state stays as it is
+int launch_parallel_step(const WindowArgs *w, float *wout, const LightningArgs *l, float *lout, const ParallelWork &work,
+                         const int *tokpos, const int *ctrl);
+
 // ---- attention of prompt rows with key and value heads of different sizes (attn_rows_*.hip) ----
 struct AttnRowsArgs {
   float *out;             // (S, H x dv), ldo floats apart
@@ -68,6 +123,8 @@ struct AttnRowsArgs {
   float scale;
   const float *sink;      // [H] or null
   const float *gate;      // (S, H x dv) rows ldg apart or null: the output is multiplied by its sigmoid
+  int window;             // > 0: a row sees its last `window` keys only, itself included
+  float out_scale = 1.0f; // a factor of the output
 };
 int launch_attn_rows(const AttnRowsArgs &a, bool fp32_operands);
 int launch_attn_rows_f32(const AttnRowsArgs &a);
@@ -86,6 +143,12 @@ int launch_sinusoid_table(float *table, int rows, int dim, double base);
 int launch_place_taps(float *dst, const float *w, int channels, int taps, int C, int ch0, int hr, int hrp);
 int launch_neg_exp(float *y, const float *x, int n);
 int launch_softcap(float *y, int64_t n, float cap);
+// x[i] += 1 for a norm weight that is stored around zero
+int launch_add_one(float *x, int n);
+// table[p][i] = (cos, sin)(p freqs[i]) * mscale, computed in double precision
+int launch_rope_table(float2 *table, const double *freqs, int rows, int half, double mscale);
+// x[t] += wte[ids[t]] (+ wpe[pos[0] + t]) for `ntok` rows of n floats (an id outside the vocabulary selects no row)
+int launch_add_embedding(float *x, const float *wte, const float *wpe, const int *ids, const int *pos, int ntok, int vocab, int n, int max_pos);
 // dst[i] = src[rows[i]] for rows of n floats
 int launch_gather_rows(float *dst, const float *src, const int *rows, int nrows, int n);
 

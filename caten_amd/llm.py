@@ -199,11 +199,16 @@ def make_llama(cfg: dict, state_dict: Dict[str, Tensor], device: int = 0) -> Tra
 
 class MixedTransformer(Transformer):
     """A decoder whose layers are listed one by one (cthip_decoder_create_mixed).  cfg: `vocab`, `dim`, `max_seq`, `eps`,
-    `norm` ("layernorm" or "rmsnorm"), `position_base`, `logit_softcap` (0 = none), `precision` (operand format of the
-    products over several rows, None = the library's option) and `layers`, each a dict of `mixer` ("delta" or
-    "latent"), that mixer's sizes and `ffn` (0 = none)."""
+    `norm` ("layernorm" or "rmsnorm"), `norm_plus_one` (norm weights stored around zero), `position_base`, `logit_softcap`
+    (0 = none), `tied_head`, `loop` ((start, stop, times) of the layers that run several times, None = none), `precision`
+    (operand format of the products over several rows, None = the library's option) and `layers`, each a dict of `mixer`
+    ("delta", "latent", "window" or "lightning") and that mixer's sizes, or `mixers`, a list of two such dicts side by
+    side, and of `ffn` (0 = none), `glu` ((alpha, limit, shift) of the gated unit, None = SwiGLU) and `layer_scale`.
+    A window mixer's `rot`: None or a dict of `dims`, `base` and, for YaRN, `factor`, `original`, `fast`, `slow`; its
+    `sink`: None, "tensor" or "zero".  A lightning mixer's `decay`: one factor per head."""
 
-    MIXERS = {"delta": _lib.MIXER_DELTA, "latent": _lib.MIXER_LATENT}
+    MIXERS = {"delta": _lib.MIXER_DELTA, "latent": _lib.MIXER_LATENT, "window": _lib.MIXER_WINDOW, "lightning": _lib.MIXER_LIGHTNING}
+    SINKS = {None: _lib.SINK_NONE, False: _lib.SINK_NONE, True: _lib.SINK_TENSOR, "tensor": _lib.SINK_TENSOR, "zero": _lib.SINK_ZERO}
     NORMS = {"layernorm": _lib.PRO_LAYERNORM, "rmsnorm": _lib.PRO_RMSNORM}
 
     def __init__(self, cfg: dict, device: int = 0):
@@ -215,13 +220,36 @@ class MixedTransformer(Transformer):
         c.norm, c.eps = self.NORMS[cfg.get("norm", "layernorm")], cfg["eps"]
         c.position_base, c.logit_softcap = cfg.get("position_base") or 0.0, cfg.get("logit_softcap") or 0.0
         c.precision = -1 if cfg.get("precision") is None else cfg["precision"]
+        c.norm_plus_one, c.tied_head = int(cfg.get("norm_plus_one", False)), int(cfg.get("tied_head", False))
+        c.loop_start, c.loop_stop, c.loop_times = cfg.get("loop") or (0, 0, 1)
         layers = (_lib.LayerSpec * len(cfg["layers"]))()
-        for s, l in zip(layers, cfg["layers"]):
-            s.mixer, s.heads, s.dim, s.vdim = self.MIXERS[l["mixer"]], l["heads"], l["dim"], l["vdim"]
-            s.kv_heads, s.conv = l.get("kv_heads", l["heads"]), l.get("conv", 0)
-            s.kv_rank, s.scale = l.get("kv_rank", 0), l.get("scale", 0.0)
-            s.sink, s.gate, s.ffn = int(l.get("sink", False)), int(l.get("gate", False)), l.get("ffn") or 0
+        for y, l in zip(layers, cfg["layers"]):
+            mixers = l.get("mixers") or [l]
+            if len(mixers) > 2:
+                raise ValueError(f"a layer has one mixer or two side by side, not {len(mixers)}")
+            y.n_mixers, y.ffn = len(mixers), l.get("ffn") or 0
+            y.glu_alpha, y.glu_limit, y.glu_shift = l.get("glu") or (1.0, float("inf"), 0.0)
+            y.layer_scale = int(l.get("layer_scale", False))
+            for s, m in zip(y.mixers, mixers):
+                self._mixer(s, m)
         _lib.check(self.lib.cthip_decoder_create_mixed(C.byref(self.handle), C.byref(c), layers))
+
+    def _mixer(self, s, m: dict) -> None:
+        s.mixer, s.heads, s.dim, s.vdim = self.MIXERS[m["mixer"]], m["heads"], m["dim"], m["vdim"]
+        s.kv_heads, s.conv = m.get("kv_heads", m["heads"]), m.get("conv", 0)
+        s.kv_rank, s.scale = m.get("kv_rank", 0), m.get("scale", 0.0)
+        s.sink, s.gate = self.SINKS[m.get("sink")], int(m.get("gate", False))
+        s.window, s.bias, s.qk_norm = m.get("window", 0), int(m.get("bias", False)), int(m.get("qk_norm", False))
+        s.out_scale = m.get("out_scale", 1.0)
+        rot = m.get("rot")
+        if rot:
+            s.rot_dims, s.rot_base = rot["dims"], rot["base"]
+            s.rot_factor, s.rot_original = rot.get("factor", 0.0), rot.get("original", 0.0)
+            s.rot_fast, s.rot_slow = rot.get("fast", 0.0), rot.get("slow", 0.0)
+        if m["mixer"] == "lightning":
+            if len(m["decay"]) != m["heads"]:
+                raise ValueError(f"{len(m['decay'])} decays for {m['heads']} heads")
+            s.decay = (C.c_double * m["heads"])(*m["decay"])  # (the structure keeps it alive)
 
 
 def zuselix_config(config: dict) -> dict:
@@ -244,8 +272,32 @@ def zuselix_config(config: dict) -> dict:
                 logit_softcap=config.get("logit_softcap") or 0.0, layers=layers)
 
 
+def matalix_config(config: dict) -> dict:
+    """config.json of a Matalix model -> MixedTransformer's cfg (without max_seq)"""
+    layers = []
+    for i, l in enumerate(config["layers"]):
+        if l["type"] != "parallel":
+            raise ValueError(f"layer {i}: mixer type {l['type']!r} is not part of this design")
+        m, mlp = l["mixer"], l.get("mlp")
+        left = {k: m["left"][k] for k in ("heads", "kv_heads", "dim", "vdim", "scale")}
+        rot = m["left"]["rot"]
+        left.update(mixer="window", window=m["left"]["mask"]["size"], rot=dict(dims=rot["dims"], base=rot["base"], **(rot.get("scaling") or {})),
+                    bias=True, qk_norm=True, sink="zero", gate=True, out_scale=m["left_scale"])
+        right = {k: m["right"][k] for k in ("heads", "dim", "vdim", "decay")}
+        right.update(mixer="lightning", out_scale=m["right_scale"])
+        layer = dict(mixers=[left, right], layer_scale=True)
+        if mlp is not None:
+            if mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: a feed-forward of kind {mlp['kind']!r} is not part of this design")
+            layer.update(ffn=int(mlp["ff"]), glu=(1.702, mlp["limit"], 1.0))
+        layers.append(layer)
+    loop = config.get("loop")
+    return dict(vocab=config["vocab"], dim=config["width"], eps=config["norm"]["eps"], norm="rmsnorm", norm_plus_one=True, tied_head=True,
+                loop=(loop["start"], loop["stop"], loop["times"]) if loop else None, layers=layers)
+
+
 # architecture name of a model directory's config.json -> (its configuration, the session's class)
-ARCHITECTURES = {"Zuselix": (zuselix_config, MixedTransformer)}
+ARCHITECTURES = {"Matalix": (matalix_config, MixedTransformer), "Zuselix": (zuselix_config, MixedTransformer)}
 
 
 def load_model(path: str, dtype: str = "bfloat16", max_seq: int = 2048, device: int = 0) -> Transformer:

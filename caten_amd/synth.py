@@ -153,6 +153,58 @@ def zuselix_tensor(name: str, shape: tuple, rng) -> np.ndarray:
     return a if name == "embed" else a / np.float32(np.sqrt(shape[-1]))
 
 
+def _matalix(width, ff, heads, kv_heads, window, layers, loop, vocab=32000):
+    """heads of 128; as many lightning heads of 128 as half the query heads, decays of tens to thousands of tokens"""
+    n = heads // 2
+    left = dict(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, scale=128 ** -0.5, mask={"size": window},
+                rot=dict(base=10000.0, dims=128, scaling=dict(factor=4.0, original=2048, fast=32.0, slow=1.0)))
+    right = dict(heads=n, dim=128, vdim=128, decay=[1.0 - 2.0 ** -(4.0 + 6.0 * h / max(n - 1, 1)) for h in range(n)])
+    layer = {"type": "parallel", "mixer": dict(left=left, left_scale=0.7, right=right, right_scale=0.6), "mlp": {"kind": "dense", "ff": ff, "limit": 7.0}}
+    return {"architecture": "Matalix", "layers": [layer] * layers, "loop": loop, "norm": {"eps": 1e-5}, "vocab": vocab, "width": width}
+
+
+# config.json-shaped configurations beside Llama shapes of the same width, feed-forward, layer runs, heads and vocabulary
+MATALIX_CONFIGS = {
+    "matalix-1b": _matalix(2048, 5632, 16, 4, 1024, 16, dict(start=5, stop=11, times=2)),  # (22 layer runs)
+    "matalix-7b": _matalix(4096, 11008, 32, 8, 2048, 12, dict(start=4, stop=8, times=2)),  # (16 layer runs)
+}
+
+
+def matalix_shapes(config: dict) -> dict:
+    """tensor name -> shape of a Matalix model (cthip_decoder_create_mixed's state-dict keys)"""
+    W, V = config["width"], config["vocab"]
+    out = {"embed": (V, W), "final.norm": (W,)}
+    for i, layer in enumerate(config["layers"]):
+        p, a, b = f"l{i}.", layer["mixer"]["left"], layer["mixer"]["right"]
+        q, k, v, o = a["heads"] * a["dim"], a["kv_heads"] * a["dim"], a["kv_heads"] * a["vdim"], a["heads"] * a["vdim"]
+        qk, ro = b["heads"] * b["dim"], b["heads"] * b["vdim"]
+        out.update({p + "norm1": (W,), p + "ls1": (W,)})
+        out.update({p + "mix.left." + n: s for n, s in {
+            "q": (q, W), "q.b": (q,), "q.norm": (q,), "k": (k, W), "k.b": (k,), "k.norm": (k,), "v": (v, W), "v.b": (v,), "g": (o, W), "o": (W, o)}.items()})
+        out.update({p + "mix.right." + n: s for n, s in {
+            "q": (qk, W), "k": (qk, W), "v": (ro, W), "g": (ro, W), "norm": (ro,), "o": (W, ro)}.items()})
+        if layer["mlp"] is not None:
+            F = layer["mlp"]["ff"]
+            out.update({p + "norm2": (W,), p + "ls2": (W,), p + "mlp.gate": (F, W), p + "mlp.up": (F, W), p + "mlp.down": (W, F)})
+    return out
+
+
+def matalix_tensor(name: str, shape: tuple, rng) -> np.ndarray:
+    """one tensor's random fp32 values: unit-variance sums, norms stored around zero or one as the design has them, layer
+    scales around a half, biases that show"""
+    last = name.rsplit(".", 1)[-1]
+    a = rng.standard_normal(shape, dtype=np.float32)
+    if last in ("norm1", "norm2") or name == "final.norm":
+        return 0.2 * a
+    if last == "norm":
+        return 1.0 + 0.2 * a
+    if last in ("ls1", "ls2"):
+        return 0.5 + 0.15 * a
+    if last == "b":
+        return 0.3 * a
+    return a if name == "embed" else a / np.float32(np.sqrt(shape[-1]))
+
+
 def prompt(vocab: int, length: int = 16, seed: int = 0) -> list:
     rng = np.random.default_rng(seed + 1000)
     return [int(t) for t in rng.integers(0, vocab, size=length)]

@@ -368,30 +368,62 @@ typedef struct {
 int cthip_decoder_create(void **dec, const cthip_decoder_config *cfg);
 int cthip_decoder_destroy(void *dec);
 
-/* A decoder whose layers are listed one by one, each with a token mixer and its sizes and, optionally, a SwiGLU
- * feed-forward.  Pre-norm: x += mixer(norm1(x)), then x += ff(norm2(x)).  Such a session keeps, besides what a
- * latent-attention layer caches, recurrent state that only moves forward: a forward starts at position 0 (a new
- * sequence) or where the last one ended.  State-dict keys (i = layer; [rows, cols] as stored, y = W x):
- *   embed [vocab, dim], final.norm, head [vocab, dim], l<i>.norm1, l<i>.norm2,
- *   l<i>.mlp.gate / .up [ffn, dim], .down [dim, ffn]
+/* A decoder whose layers are listed one by one, each with one token mixer, or two side by side that read the same input,
+ * their sizes and, optionally, a gated feed-forward.  Pre-norm: x += mixer(norm1(x)), then x += ff(norm2(x)); layers
+ * loop_start .. loop_stop - 1 may run several times in a row with the same weights, each run with a cache or state of
+ * its own.  Such a session keeps, besides what attention layers cache, recurrent state that only moves forward: a
+ * forward starts at position 0 (a new sequence) or where the last one ended.  State-dict keys (i = layer; [rows, cols]
+ * as stored, y = W x):
+ *   embed [vocab, dim], final.norm, head [vocab, dim] (unless tied_head), l<i>.norm1, l<i>.norm2,
+ *   l<i>.mlp.gate / .up [ffn, dim], .down [dim, ffn]; with layer_scale l<i>.ls1, l<i>.ls2 [dim]
+ *   one mixer: l<i>.mix.*; two of them: l<i>.mix.left.* and l<i>.mix.right.*, each with the keys of its kind
  *   CTHIP_MIXER_DELTA (gated delta rule): l<i>.mix.q / .k [kv_heads dim, width], .v [heads vdim, width], each with
  *     .conv [channels, conv] (last column: the current token), .b / .a [heads, width], .A_log, .dt_bias [heads],
  *     .g [heads vdim, width], .norm [vdim], .o [width, heads vdim]
  *   CTHIP_MIXER_LATENT (attention over a cached latent): l<i>.mix.q [heads dim, width], .dkv [kv_rank, width],
  *     .dkv.norm [kv_rank], .uk [heads dim, kv_rank], .uv [heads vdim, kv_rank], .o [width, heads vdim] and, where the
  *     layer has them, .sink [heads] and .g [heads vdim, width]
+ *   CTHIP_MIXER_WINDOW (grouped-query attention over the last `window` positions): .q [heads dim, width], .k [kv_heads
+ *     dim, width], .v [kv_heads vdim, width], .o [width, heads vdim] and, where the layer has them, .q.b, .k.b, .v.b
+ *     (biases), .q.norm, .k.norm (weights of an RMS norm over the whole projection), .sink [heads], .g [heads vdim, width]
+ *   CTHIP_MIXER_LIGHTNING (linear attention, S <- decay S + k v^T, o = S^T q with q, k, v behind silu): .q / .k [heads dim,
+ *     width], .v / .g [heads vdim, width], .norm [heads vdim] (RMS norm over the concatenated heads), .o [width, heads vdim]
  * Linear weights are fp32, fp16 or bf16, one format per session. */
 #define CTHIP_MIXER_DELTA 0
 #define CTHIP_MIXER_LATENT 1
+#define CTHIP_MIXER_WINDOW 2
+#define CTHIP_MIXER_LIGHTNING 3
+#define CTHIP_SINK_TENSOR 1
+#define CTHIP_SINK_ZERO 2
 typedef struct {
   int mixer;           /* CTHIP_MIXER_* */
-  int heads, kv_heads; /* kv_heads: query / key heads of a delta layer, each shared by heads / kv_heads value heads */
+  int heads, kv_heads; /* kv_heads: query / key heads of a delta layer, each shared by heads / kv_heads value heads; key /
+                          value heads of a window layer, each shared by heads / kv_heads query heads */
   int dim, vdim;       /* per head: query / key size, value size (at most 256) */
   int conv;            /* delta: taps of the short convolutions */
   int kv_rank;         /* latent: size of the cached vector (at most 1024) */
-  float scale;         /* latent: the scores' factor */
-  int sink, gate;      /* latent: 1 = the softmax has a sink / the output is gated */
-  int ffn;             /* feed-forward size, 0 = none */
+  float scale;         /* latent, window: the scores' factor */
+  int sink;            /* latent, window: one more term of the softmax's denominator, without a value: 0 = none,
+                          CTHIP_SINK_TENSOR = a learned logit per head, CTHIP_SINK_ZERO (window) = a logit of 0 */
+  int gate;            /* latent, window: 1 = the output is multiplied by sigmoid(.g x) */
+  int window;          /* window: position i sees j with 0 <= i - j < window */
+  int bias, qk_norm;   /* window: 1 = the projections have biases / queries and keys an RMS norm */
+  int rot_dims;        /* window: rotated entries of a head (even, 0 = none): entries i and i + rot_dims / 2 are a pair */
+  double rot_base;
+  /* rot_factor > 0: YaRN.  Pairs that turn fewer than rot_slow times over rot_original positions are stretched by
+   * rot_factor, those that turn more than rot_fast times are not, with a ramp between; cosine and sine are multiplied
+   * by 0.1 ln(rot_factor) + 1 */
+  double rot_factor, rot_original, rot_fast, rot_slow;
+  const double *decay; /* lightning: `heads` factors in 0 .. 1, read by the create call */
+  float out_scale;     /* window, lightning: the mixer's result is multiplied by this */
+} cthip_mixer_spec;
+typedef struct {
+  int n_mixers;        /* 1, or 2 side by side (window and lightning only) */
+  cthip_mixer_spec mixers[2];
+  int ffn;             /* feed-forward size, 0 = none: down (g sigmoid(glu_alpha g) (u + glu_shift)) with g = min(gate x,
+                          glu_limit), u = up x held within -glu_limit .. glu_limit */
+  float glu_alpha, glu_limit, glu_shift; /* 1, infinity, 0 = SwiGLU */
+  int layer_scale;     /* 1 = mixer and feed-forward results are multiplied by .ls1 / .ls2 before they are added */
 } cthip_layer_spec;
 typedef struct {
   int n_layers, dim, vocab, max_seq;
@@ -400,6 +432,10 @@ typedef struct {
   float position_base; /* > 0: a sinusoidal position vector of this base is added to the embedding */
   float logit_softcap; /* > 0: logits = cap tanh(logits / cap) */
   int precision;       /* operand format of the products over several rows, as option "gemm_precision"; -1 = that option */
+  int norm_plus_one;   /* 1 = norm1, norm2 and final.norm are stored around zero: their weights are 1 + w */
+  int tied_head;       /* 1 = the logits are products with the embedding table */
+  int loop_start, loop_stop, loop_times; /* layers start .. stop - 1 run loop_times times in a row; before every pass but
+                          the first the embedding is added to the residual stream.  loop_times <= 1 = once */
 } cthip_mixed_config;
 int cthip_decoder_create_mixed(void **dec, const cthip_mixed_config *cfg, const cthip_layer_spec *layers);
 /* load-state-dict (source/api/module.lisp:290-320): hands one tensor to the
@@ -448,8 +484,9 @@ int cthip_decoder_layer_launches(void *dec);
  * cache their dequantised values, in a buffer the next peek overwrites), "logits", "x"; with a Q8_0 cache also
  * the planes themselves, "k_cache_q8.<l>" / "v_cache_q8.<l>" (int8[max_seq][kv_dim]) and "k_cache_d.<l>" /
  * "v_cache_d.<l>" (fp16[max_seq][kv_dim / 32]), n_floats counting their bytes in units of four.  A mixed decoder:
- * "latent.<l>" (max_seq rows of the latent, padded to a multiple of 16), "state.<l>" ([head][value column][key], both
- * padded likewise), "logits", "x". */
+ * "latent.<r>" (max_seq rows of the latent, padded to a multiple of 16), "state.<r>" ([head][value column][key], both
+ * padded likewise), "keys.<r>" / "values.<r>" (a ring of min(window, max_seq) rows of kv_heads padded heads, position p in
+ * row p mod rows), "logits", "x"; r counts layer runs (a looped layer's every pass by itself). */
 int cthip_decoder_peek(void *dec, const char *what, void **ptr, int64_t *n_floats);
 
 /* ================================================================== */

@@ -142,7 +142,7 @@ def test_configuration():
 
 def test_registry(tmp_path):
     (tmp_path / "config.json").write_text(json.dumps({"architecture": "Other"}))
-    with pytest.raises(ValueError, match="'Other' is not registered .known: Zuselix"):
+    with pytest.raises(ValueError, match="'Other' is not registered .known: Matalix, Zuselix"):
         llm.load_model(str(tmp_path))
     (tmp_path / "config.json").write_text(json.dumps(mm.config([mm.delta()])))
     with pytest.raises(ValueError, match="dtype 'int8'"):
