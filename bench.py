@@ -384,7 +384,7 @@ def main():
                     help="also run one 256 MiB device-to-device copy (a kernel of known traffic to scale "
                          "rocprofv3 FETCH_SIZE / WRITE_SIZE readings by)")
     ap.add_argument("--mixed", nargs="*", metavar="SIZE", default=None,
-                    help="instead of the headline workload: Zuselix shapes beside Llama shapes of equal size (bench_mixed.py)")
+                    help="instead of the headline workload: Zuselix and Matalix shapes beside Llama shapes of equal size (bench_mixed.py)")
     args = ap.parse_args()
     if args.mixed is not None:
         import bench_mixed

@@ -1,7 +1,8 @@
 #!/usr/bin/env python3
-"""Zuselix-shaped models (gated delta rule and latent attention layers) beside Llama shapes of the same width, feed-forward,
-depth and vocabulary, both with bf16 weights, on one MI355X: greedy decode at short and long contexts and prompts as one
-batch.  `python bench.py --mixed`, or this file by itself.
+"""Zuselix shapes (gated delta rule and latent attention layers) and Matalix shapes (sliding-window attention beside lightning
+attention, some layers run twice) beside Llama shapes of the same width, feed-forward, layer runs, heads and vocabulary, all
+with bf16 weights, on one MI355X: greedy decode at short and long contexts and prompts as one batch.
+`python bench.py --mixed`, or this file by itself.
 
 Weights are synthetic; one layer of each kind is drawn and loaded into every layer of that kind, each with its own copy in
 HBM.  A session's figures are reported only after its logits for a prompt in one forward agree with the same prompt token
@@ -22,33 +23,57 @@ import numpy as np
 HBM_PEAK_GBS = 8000.0
 
 
-def zuselix_session(name: str, max_seq: int):
-    """(session, cfg, GFLOP of the Linear layers per token, head left out)"""
+def designs() -> dict:
+    """name -> (sizes, tensor shapes, random tensor, configuration of a session)"""
     from caten_amd import llm, synth
+    return {"zuselix": (synth.ZUSELIX_CONFIGS, synth.zuselix_shapes, synth.zuselix_tensor, llm.zuselix_config),
+            "matalix": (synth.MATALIX_CONFIGS, synth.matalix_shapes, synth.matalix_tensor, llm.matalix_config)}
+
+
+def sizes() -> list:
+    return [n for d in designs().values() for n in d[0]]
+
+
+def design_of(name: str) -> str:
+    return next(k for k, d in designs().items() if name in d[0])
+
+
+def layer_runs(config: dict) -> list:
+    """how often each layer runs per token"""
+    loop = config.get("loop") or {"start": 0, "stop": 0, "times": 1}
+    return [loop["times"] if loop["start"] <= i < loop["stop"] else 1 for i in range(len(config["layers"]))]
+
+
+def mixed_session(name: str, max_seq: int):
+    """(session, cfg, GFLOP of the Linear layers per token, head left out)"""
+    from caten_amd import llm
     from caten_amd.quant import to_bf16
-    config = synth.ZUSELIX_CONFIGS[name]
-    rng = np.random.default_rng(0)
+    configs, shapes, tensor, to_cfg = designs()[design_of(name)]
+    config = configs[name]
+    rng, runs = np.random.default_rng(0), layer_runs(config)
     drawn, sd, flop = {}, {}, 0.0
-    for key, shape in synth.zuselix_shapes(config).items():
+    for key, shape in shapes(config).items():
         layer, _, rest = key.partition(".")
-        kind = config["layers"][int(layer[1:])]["type"] + "." + rest if layer[1:].isdigit() else key
+        in_layer = layer[1:].isdigit()
+        kind = config["layers"][int(layer[1:])]["type"] + "." + rest if in_layer else key
         if kind not in drawn:
-            bits = to_bf16(synth.zuselix_tensor(key, shape, rng).ravel())
+            bits = to_bf16(tensor(key, shape, rng).ravel())
             rows, cols = shape if len(shape) == 2 else (1, shape[0])
             drawn[kind] = llm.Tensor("bf16", bits.view(np.uint8), rows, cols)
         sd[key] = drawn[kind]
-        if len(shape) == 2 and shape[1] >= 16 and key not in ("embed", "head"):
-            flop += 2.0 * shape[0] * shape[1]
-    cfg = dict(llm.zuselix_config(config), max_seq=max_seq)
+        if in_layer and len(shape) == 2 and shape[1] >= 16:
+            flop += 2.0 * shape[0] * shape[1] * runs[int(layer[1:])]
+    cfg = dict(to_cfg(config), max_seq=max_seq)
     return llm.MixedTransformer(cfg).load_state_dict(sd), cfg, flop / 1e9
 
 
 def llama_session(name: str, max_seq: int):
-    """the Llama shape of the same width, feed-forward, depth, heads and vocabulary"""
+    """the Llama shape of the same width, feed-forward, layer runs, heads and vocabulary"""
     from caten_amd import llm, synth
-    z = synth.ZUSELIX_CONFIGS[name]
+    z = designs()[design_of(name)][0][name]
     m = z["layers"][0]["mixer"]
-    cfg = dict(n_layers=len(z["layers"]), dim=z["width"], n_heads=m["heads"], n_kv_heads=m["kv_heads"], ffn=z["layers"][0]["mlp"]["ff"],
+    m = m.get("left", m)
+    cfg = dict(n_layers=sum(layer_runs(z)), dim=z["width"], n_heads=m["heads"], n_kv_heads=m["kv_heads"], ffn=z["layers"][0]["mlp"]["ff"],
                vocab=z["vocab"], max_seq=max_seq, eps=1e-5, rope_base=10000.0)
     one = llm.llama_state_dict(synth.llama_weights(dict(cfg, n_layers=1), seed=0, threads=8), "bf16", threads=8)
     sd = {}
@@ -105,7 +130,7 @@ def measure(name: str, kind: str, prompts=(512, 2048), contexts=(16, 1900), step
     lib = _lib.init()
     max_seq = max([c + steps + 16 for c in contexts] + list(prompts) + [64])
     t0 = time.perf_counter()
-    model, cfg, gflop = (zuselix_session if kind == "zuselix" else llama_session)(name, max_seq)
+    model, cfg, gflop = (llama_session if kind == "llama" else mixed_session)(name, max_seq)
     err = agree(model, cfg["vocab"])
     if not err < 2e-2:
         raise SystemExit(f"bench_mixed: {kind} {name}: prompt and decode logits differ by {err:.3g}; no figure is reported")
@@ -124,19 +149,18 @@ def measure(name: str, kind: str, prompts=(512, 2048), contexts=(16, 1900), step
     return res
 
 
-def main(names=None, kinds=("zuselix", "llama"), **measured) -> None:
-    from caten_amd import synth
-    for name in names or list(synth.ZUSELIX_CONFIGS):
-        if name not in synth.ZUSELIX_CONFIGS:
-            raise SystemExit(f"bench_mixed: unknown size {name} (known: {', '.join(synth.ZUSELIX_CONFIGS)})")
+def main(names=None, kinds=("own", "llama"), **measured) -> None:
+    for name in names or sizes():
+        if name not in sizes():
+            raise SystemExit(f"bench_mixed: unknown size {name} (known: {', '.join(sizes())})")
         for kind in kinds:
-            print(json.dumps(measure(name, kind, **measured)), flush=True)
+            print(json.dumps(measure(name, design_of(name) if kind == "own" else kind, **measured)), flush=True)
 
 
 if __name__ == "__main__":
     ap = argparse.ArgumentParser()
     ap.add_argument("--sizes", default="")
-    ap.add_argument("--kinds", default="zuselix,llama")
+    ap.add_argument("--kinds", default="own,llama", help="own: the size's design")
     ap.add_argument("--contexts", default="16,1900", help="prompt lengths in front of the timed decode steps")
     ap.add_argument("--prompts", default="512,2048", help="timed prompt lengths")
     ap.add_argument("--steps", type=int, default=64)
