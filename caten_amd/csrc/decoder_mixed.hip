@@ -695,7 +695,7 @@ int mixed_prefill(Decoder *d, float *X, float *XN, const int *ids, int s, int n)
           case CTHIP_MIXER_DELTA: rc = launch_delta_rows(delta_of(br, r.keep[b], P), O, s, n, W); break;
           case CTHIP_MIXER_LATENT: rc = latent_rows(br, r.keep[b], L.out->cols); break;
           case CTHIP_MIXER_WINDOW: rc = window_rows(br, r.keep[b], L.out->cols); break;
-          default: rc = launch_lightning_rows(lightning_of(br, r.keep[b], P), P + br.row0, O + br.col0, L.out->cols, s, n, W);
+          default: rc = launch_lightning_rows(lightning_of(br, r.keep[b], P), O + br.col0, L.out->cols, s, n, W);
         }
         if (rc) return rc;
       }

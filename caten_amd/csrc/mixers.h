@@ -93,18 +93,17 @@ struct LightningArgs {
   float eps, out_scale;
   float *S;                // [H][DV][DK], fp32
 };
-// s tokens at positions n .. n + s - 1 -> out rows ldo floats apart; p: the projection rows, q, k and v of which pass silu
-// in place; scratch: lightning_scratch_floats() floats
+// s tokens at positions n .. n + s - 1 -> out rows ldo floats apart; scratch: lightning_scratch_floats() floats
 size_t lightning_scratch_floats(const LightningArgs &a, int s);
-int launch_lightning_rows(const LightningArgs &a, float *p, float *out, int64_t ldo, int s, int n, float *scratch);
+int launch_lightning_rows(const LightningArgs &a, float *out, int64_t ldo, int s, int n, float *scratch);
 
 // ---- a decode step of either, or of both side by side in one launch ----
 struct ParallelWork {
   float *part;   // window: every key range's unnormalised sums, maximum and denominator
   int *count;    // tickets: one for the lightning heads, then window_tickets() of them; zeroed (each launch leaves them zeroed again)
-  float *raw;    // lightning: H x DV outputs before the norm, then a sum of squares per workgroup
+  float *raw;    // lightning: H x DV outputs before the norm
 };
-constexpr int kWindowMaxRanges = 16;
+constexpr int kWindowMaxRanges = 32;
 int window_tickets(const WindowArgs &a);
 size_t window_part_floats(const WindowArgs &a);
 size_t lightning_raw_floats(const LightningArgs &a);

@@ -3,40 +3,62 @@
 //
 //   window     workgroup (key range, key/value head, up to QB of its query heads).  It takes the root mean squares of all
 //              queries and keys, normalises and rotates its own, and attends over its share of the ring: 16 lanes per row,
-//              16 rows a tile, range r of n takes tiles r, r + n, ... .  Rings are walked by row, not by position, so the
+//              16 rows a tile, range r takes the r-th run of `2^lper` tiles.  Rings are walked by row, not by position, so the
 //              first rows are asked for before the position is known; which position a row holds follows from it.  The new
-//              key and value come from the projection row; the range that owns their row of the ring stores them.
+//              key and value come from the projection row; the range that owns their row of the ring stores them.  While
+//              few rows are held, few ranges have any, and a single one finishes by itself.  Every group of 16 lanes keeps a
+//              softmax of its own; they meet in LDS.
 //   lightning  workgroup (head, 16 value columns), 16 lanes per column: the state's rows are read once, updated, read out
 //              and written once.  The norm takes all heads' outputs.
 //
 // What meets across workgroups -- a head's key ranges, the heads' outputs in front of the norm -- is left in memory with
 // device-scope stores, a ticket is drawn, and the workgroup with the last ticket finishes (as k_attn_cached does).
+#include <type_traits>
+
 #include "common.h"
 #include "mixers.h"
 
 namespace cthip {
 
+constexpr int kWindowTiles = 4;  // tiles of a key range, at least
 struct WindowShape {
-  int ranges, qgroups, blocks;  // qgroups: workgroups of up to QB query heads per key/value head
+  int ranges, lper;  // key ranges of 2^lper tiles each
+  int rep, qgroups;  // query heads per key/value head; workgroups of up to QB of them
+  unsigned inv;      // about 2^32 / rows
+  int blocks() const { return ranges * heads; }
+  int heads;         // workgroups of a range
 };
-constexpr int window_qb(int rep) { return rep >= 3 ? 4 : rep; }
+static int window_pieces(const WindowArgs &a) { return ((a.DK > a.DV ? a.DK : a.DV) + 63) / 64; }
+static int window_qb(const WindowArgs &a) {  // (heads past 128 entries: what two of them keep fits LDS)
+  const int rep = a.H / a.G;
+  return rep >= 3 && window_pieces(a) <= 2 ? 4 : rep >= 2 ? 2 : 1;
+}
 static WindowShape window_shape(const WindowArgs &a) {
-  const int rep = a.H / a.G, qb = window_qb(rep);
   WindowShape w;
-  w.qgroups = (rep + qb - 1) / qb;
-  const int tiles = (a.rows + 15) / 16, fill = 512 / (a.G * w.qgroups);
-  w.ranges = tiles < kWindowMaxRanges ? tiles : kWindowMaxRanges;
-  if (w.ranges > fill) w.ranges = fill < 1 ? 1 : fill;
-  w.blocks = w.ranges * w.qgroups * a.G;
+  w.rep = a.H / a.G;
+  w.qgroups = (w.rep + window_qb(a) - 1) / window_qb(a);
+  w.heads = a.G * w.qgroups;
+  const int tiles = (a.rows + 15) / 16, fill = 512 / w.heads;
+  const int most = fill < 1 ? 1 : fill < kWindowMaxRanges ? fill : kWindowMaxRanges;
+  for (w.lper = 0; (1 << w.lper) < kWindowTiles || ((tiles - 1) >> w.lper) + 1 > most; w.lper++) {}
+  w.ranges = ((tiles - 1) >> w.lper) + 1;
+  w.inv = a.rows > 1 ? (unsigned)((1ull << 32) / (unsigned)a.rows) : 0xffffffffu;
   return w;
 }
 constexpr int part_pitch(int dv) { return dv + 4; }  // a range's record of one head: DV sums, maximum, denominator, two unused
-int window_tickets(const WindowArgs &a) { return window_shape(a).qgroups * a.G; }
-size_t window_part_floats(const WindowArgs &a) { return (size_t)window_shape(a).blocks * window_qb(a.H / a.G) * part_pitch(a.DV); }
-size_t lightning_raw_floats(const LightningArgs &a) { return (size_t)a.H * a.DV + (size_t)a.H * a.DV / 16; }
+int window_tickets(const WindowArgs &a) { return window_shape(a).heads; }
+size_t window_part_floats(const WindowArgs &a) { return (size_t)window_shape(a).blocks() * window_qb(a) * part_pitch(a.DV); }
+size_t lightning_raw_floats(const LightningArgs &a) { return (size_t)a.H * a.DV; }
 
 __device__ __forceinline__ float agent_load(const float *p) { return __hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
 __device__ __forceinline__ void agent_store(float *p, float v) { __hip_atomic_store(p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
+// two floats at an address that is a multiple of 8
+__device__ __forceinline__ float2 agent_load2(const float *p) {
+  return __builtin_bit_cast(float2, __hip_atomic_load((const unsigned long long *)p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
+}
+__device__ __forceinline__ void agent_store2(float *p, float2 v) {
+  __hip_atomic_store((unsigned long long *)p, __builtin_bit_cast(unsigned long long, v), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+}
 
 // true in the workgroup that draws the last of `n` tickets; every thread's stores have reached memory by then
 __device__ __forceinline__ bool last_ticket(int *count, int n, int *lds) {
@@ -52,23 +74,46 @@ __device__ __forceinline__ bool last_ticket(int *count, int n, int *lds) {
 template <int NC, int QB>
 struct StepLds {
   float q[QB][64 * NC], k[64 * NC];
-  float o[4][QB][64 * NC], m[4][QB], l[4][QB];
+  float o[16][QB][64 * NC], m[16][QB], l[16][QB];  // of every group of 16 lanes
   float red[8];
   int ticket;
 };
 
 // NC: 64-entry pieces of a head, at most; QB: query heads of a workgroup
 template <int NC, int QB>
-__device__ void window_step(const WindowArgs &a, int nranges, int qgroups, int block, float *__restrict__ part, int *__restrict__ count,
+__device__ void window_step(const WindowArgs &a, const WindowShape &sh, int hg, int range, float *__restrict__ part, int *__restrict__ count,
                             float *__restrict__ out, const int *__restrict__ tokpos, StepLds<NC, QB> &S) {
-  constexpr int U = NC >= 4 ? 1 : 2;  // tiles a wavefront works on together
-  constexpr int QE = (QB * 64 * NC + 255) / 256;
+  constexpr int U = NC >= 4 ? 2 : 4;  // tiles a wavefront works on together
+  constexpr int DP = 64 * NC, QE = (QB * DP + 255) / 256, SB = 4;
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, g16 = lane >> 4, l = lane & 15;
-  const int hg = block % (a.G * qgroups), range = block / (a.G * qgroups), g = hg / qgroups, rep = a.H / a.G;
-  const int h0 = g * rep + (hg % qgroups) * QB, nq = min(QB, (g + 1) * rep - h0);  // this workgroup's query heads
+  const int rep = sh.rep, g = sh.qgroups == 1 ? hg : hg / sh.qgroups, qg = hg - g * sh.qgroups;
+  const int h0 = g * rep + qg * QB, nq = min(QB, (g + 1) * rep - h0);  // this workgroup's query heads
   const int DK = a.DK, DV = a.DV, KW = a.G * DK, VW = a.G * DV, QW = a.H * DK, rows = a.rows, half = a.rope ? a.half : 0;
   const float *__restrict__ pq = a.p, *__restrict__ pk = pq + QW, *__restrict__ pv = pk + KW;
   const int pos = tokpos[1];
+  // ---- this step's queries, key and value ----
+  auto mate = [&](int d) { return d < half ? d + half : d < 2 * half ? d - half : d; };
+  auto square = [](const float4 x, float s) { return fmaf(x.x, x.x, fmaf(x.y, x.y, fmaf(x.z, x.z, fmaf(x.w, x.w, s)))); };
+  float4 x[SB], y;
+  if (a.qnorm) {
+#pragma unroll
+    for (int b = 0; b < SB; b++) x[b] = *(const float4 *)(pq + min(4 * tid + 1024 * b, QW - 4));
+    y = *(const float4 *)(pk + min(4 * tid, KW - 4));
+  }
+  float qa[QE], qb[QE], wa[QE], wb[QE];
+#pragma unroll
+  for (int j = 0; j < QE; j++) {
+    const int it = tid + 256 * j, h = min(it / DP, nq - 1), d = min(it % DP, DK - 1);
+    const int e = (h0 + h) * DK + d, f = (h0 + h) * DK + mate(d);
+    qa[j] = pq[e], qb[j] = pq[f];
+    wa[j] = a.qnorm ? a.qnorm[e] : 1.0f, wb[j] = a.qnorm ? a.qnorm[f] : 1.0f;
+  }
+  const int kd = min(tid, DK - 1);
+  const float ka = pk[g * DK + kd], kb = pk[g * DK + mate(kd)];
+  const float wka = a.knorm ? a.knorm[g * DK + kd] : 1.0f, wkb = a.knorm ? a.knorm[g * DK + mate(kd)] : 1.0f;
+  float4 vn[NC];
+#pragma unroll
+  for (int i = 0; i < NC; i++) vn[i] = *(const float4 *)(pv + g * DV + min(4 * (l + 16 * i), DV - 4));
   // ---- rows of the ring ----
   float4 kr[U][NC], vr[U][NC];
   auto request = [&](int u, int tile) {
@@ -79,53 +124,28 @@ __device__ void window_step(const WindowArgs &a, int nranges, int qgroups, int b
       vr[u][i] = *(const float4 *)(a.V + row * VW + g * DV + min(4 * (l + 16 * i), DV - 4));  // (past the head: not stored)
     }
   };
-  request(0, range);  // (whatever the position, a range starts with this tile)
-  // ---- this step's queries and key ----
-  float qa[QE], qb[QE], wa[QE], wb[QE];
+  const int first = range << sh.lper;
 #pragma unroll
-  for (int j = 0; j < QE; j++) {
-    const int it = min(tid + 256 * j, nq * DK - 1), h = it / DK, d = it - h * DK;
-    const int mate = d < half ? d + half : d < 2 * half ? d - half : d;
-    const int e = (h0 + h) * DK + d, f = (h0 + h) * DK + mate;
-    qa[j] = pq[e], qb[j] = pq[f];
-    wa[j] = a.qnorm ? a.qnorm[e] : 1.0f, wb[j] = a.qnorm ? a.qnorm[f] : 1.0f;
-  }
-  const int kd = min(tid, DK - 1), kmate = kd < half ? kd + half : kd < 2 * half ? kd - half : kd;
-  const float ka = pk[g * DK + kd], kb = pk[g * DK + kmate];
-  const float wka = a.knorm ? a.knorm[g * DK + kd] : 1.0f, wkb = a.knorm ? a.knorm[g * DK + kmate] : 1.0f;
-  float4 vn[NC];
-#pragma unroll
-  for (int i = 0; i < NC; i++) vn[i] = *(const float4 *)(pv + g * DV + min(4 * (l + 16 * i), DV - 4));
+  for (int u = 0; u < U; u++) request(u, first + u);
   float qs = 1.0f, ks = 1.0f;
   if (a.qnorm) {
-    float sq = 0.0f, sk = 0.0f;
-    constexpr int SB = 4;
-    for (int e0 = 4 * tid; e0 < QW; e0 += 1024 * SB) {
-      float4 x[SB];
+    float sq = 0.0f, sk = 4 * tid < KW ? square(y, 0.0f) : 0.0f;
 #pragma unroll
-      for (int b = 0; b < SB; b++) x[b] = *(const float4 *)(pq + min(e0 + 1024 * b, QW - 4));
-#pragma unroll
-      for (int b = 0; b < SB; b++)
-        if (e0 + 1024 * b < QW) sq = fmaf(x[b].x, x[b].x, fmaf(x[b].y, x[b].y, fmaf(x[b].z, x[b].z, fmaf(x[b].w, x[b].w, sq))));
-    }
-    for (int e = 4 * tid; e < KW; e += 1024) {
-      const float4 x = *(const float4 *)(pk + e);
-      sk = fmaf(x.x, x.x, fmaf(x.y, x.y, fmaf(x.z, x.z, fmaf(x.w, x.w, sk))));
-    }
+    for (int b = 0; b < SB; b++)
+      if (4 * tid + 1024 * b < QW) sq = square(x[b], sq);
+    for (int e = 4 * tid + 1024 * SB; e < QW; e += 1024) sq = square(*(const float4 *)(pq + e), sq);
+    for (int e = 4 * tid + 1024; e < KW; e += 1024) sk = square(*(const float4 *)(pk + e), sk);
     sq = wave_sum(sq), sk = wave_sum(sk);
     if (lane == 0) S.red[wv] = sq, S.red[4 + wv] = sk;
   }
-  const int held = min(pos + 1, rows), tiles = (held + 15) >> 4, nr = min(nranges, (tiles + 1) >> 1);
+  const int held = min(pos + 1, rows), tiles = (held + 15) >> 4, nr = ((tiles - 1) >> sh.lper) + 1;
   if (range >= nr) return;  // (uniform)
-#pragma unroll
-  for (int u = 1; u < U; u++) request(u, range + nr * u);
+  const int end = min(first + (1 << sh.lper), tiles);
   float2 qc[QE], kc = make_float2(1.0f, 0.0f);
+  auto angle = [&](int d) { return d < 2 * half ? a.rope[(int64_t)pos * half + (d < half ? d : d - half)] : make_float2(1.0f, 0.0f); };
 #pragma unroll
-  for (int j = 0; j < QE; j++) {
-    const int d = min(tid + 256 * j, nq * DK - 1) % DK, i = d < half ? d : d - half;
-    qc[j] = d < 2 * half ? a.rope[(int64_t)pos * half + i] : make_float2(1.0f, 0.0f);
-  }
-  if (kd < 2 * half) kc = a.rope[(int64_t)pos * half + (kd < half ? kd : kd - half)];
+  for (int j = 0; j < QE; j++) qc[j] = angle(min((tid + 256 * j) % DP, DK - 1));
+  kc = angle(kd);
   __syncthreads();
   if (a.qnorm) {
     qs = 1.0f / sqrtf(((S.red[0] + S.red[1]) + (S.red[2] + S.red[3])) / (float)(a.H * a.dk) + a.eps);
@@ -140,32 +160,26 @@ __device__ void window_step(const WindowArgs &a, int nranges, int qgroups, int b
     return d < half ? o0 : o1;
   };
 #pragma unroll
-  for (int j = 0; j < QE; j++) {
-    const int it = tid + 256 * j;
-    if (it < nq * DK) S.q[it / DK][it % DK] = turned(it % DK, qa[j] * qs * wa[j], qb[j] * qs * wb[j], qc[j]);
+  for (int j = 0; j < QE; j++) {  // (zero past the head and past the last query head)
+    const int it = tid + 256 * j, h = it / DP, d = it % DP;
+    if (h < QB) S.q[h][d] = h < nq && d < DK ? turned(d, qa[j] * qs * wa[j], qb[j] * qs * wb[j], qc[j]) * a.scale : 0.0f;
   }
-  if (tid < DK) S.k[tid] = turned(tid, ka * ks * wka, kb * ks * wkb, kc);
+  if (tid < DP) S.k[tid] = tid < DK ? turned(tid, ka * ks * wka, kb * ks * wkb, kc) : 0.0f;
   __syncthreads();
-  const int cur = pos % rows;
+  int cur = pos - (int)__umulhi((unsigned)pos, sh.inv) * rows;  // pos mod rows
+  while (cur >= rows) cur -= rows;
   float4 q[QB][NC], o[QB][NC], kn[NC];
   float m[QB], L[QB];
 #pragma unroll
   for (int i = 0; i < NC; i++) {
     const int e = 4 * (l + 16 * i);
-    const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
-    kn[i] = e < DK ? *(const float4 *)&S.k[e] : zero;
+    kn[i] = *(const float4 *)&S.k[e];
 #pragma unroll
-    for (int h = 0; h < QB; h++) {
-      q[h][i] = o[h][i] = zero;
-      if (h < nq && e < DK) {
-        const float4 t = *(const float4 *)&S.q[h][e];
-        q[h][i] = make_float4(t.x * a.scale, t.y * a.scale, t.z * a.scale, t.w * a.scale);
-      }
-    }
+    for (int h = 0; h < QB; h++) q[h][i] = *(const float4 *)&S.q[h][e], o[h][i] = make_float4(0.f, 0.f, 0.f, 0.f);
   }
 #pragma unroll
   for (int h = 0; h < QB; h++) m[h] = -INFINITY, L[h] = 0.0f;
-  if ((cur >> 4) % nr == range && hg % qgroups == 0 && tid < 16) {  // the new row: nobody reads this row of the ring in this step
+  if (cur >> (4 + sh.lper) == range && qg == 0 && tid < 16) {  // the new row: nobody reads this row of the ring in this step
 #pragma unroll
     for (int i = 0; i < NC; i++) {
       const int e = 4 * (l + 16 * i);
@@ -173,18 +187,18 @@ __device__ void window_step(const WindowArgs &a, int nranges, int qgroups, int b
       if (e < DV) *(float4 *)(a.V + (int64_t)cur * VW + g * DV + e) = vn[i];
     }
   }
-  for (int tile0 = range; tile0 < tiles; tile0 += U * nr) {
-    if (tile0 != range) {
+  for (int tile0 = first; tile0 < end; tile0 += U) {
+    if (tile0 != first) {
 #pragma unroll
-      for (int u = 0; u < U; u++) request(u, tile0 + nr * u);
+      for (int u = 0; u < U; u++) request(u, tile0 + u);
     }
     bool ok[U];
 #pragma unroll
     for (int u = 0; u < U; u++) {
-      const int slot = (tile0 + nr * u) * 16 + 4 * wv + g16;
+      const int slot = (tile0 + u) * 16 + 4 * wv + g16;
       int back = cur - slot;
       back += back < 0 ? rows : 0;
-      ok[u] = slot < rows && back <= pos && back < a.window;
+      ok[u] = tile0 + u < end && slot < rows && back <= pos && back < a.window;
       if (slot == cur) {
 #pragma unroll
         for (int i = 0; i < NC; i++) kr[u][i] = kn[i], vr[u][i] = vn[i];
@@ -196,7 +210,7 @@ __device__ void window_step(const WindowArgs &a, int nranges, int qgroups, int b
     }
 #pragma unroll
     for (int h = 0; h < QB; h++) {
-      float sc[U], top = -INFINITY;
+      float sc[U], m_new = m[h];
 #pragma unroll
       for (int u = 0; u < U; u++) {
         float d = 0.0f;
@@ -205,18 +219,17 @@ __device__ void window_step(const WindowArgs &a, int nranges, int qgroups, int b
           d = fmaf(q[h][i].x, kr[u][i].x, fmaf(q[h][i].y, kr[u][i].y, fmaf(q[h][i].z, kr[u][i].z, fmaf(q[h][i].w, kr[u][i].w, d))));
         d = row16_sum(d);
         sc[u] = ok[u] ? d : -INFINITY;
-        top = fmaxf(top, sc[u]);
+        m_new = fmaxf(m_new, sc[u]);
       }
-      const float m_new = fmaxf(m[h], groups16_max(top));
-      const float m_use = m_new == -INFINITY ? 0.0f : m_new;  // no row of this wavefront's yet
+      const float m_use = m_new == -INFINITY ? 0.0f : m_new;  // no row of this group's yet
       const float corr = ct_exp(m[h] - m_use);
-      float ps = 0.0f, pr[U];
+      float pr[U];
+      L[h] *= corr;
 #pragma unroll
       for (int u = 0; u < U; u++) {
         pr[u] = ct_exp(sc[u] - m_use);
-        ps += pr[u];
+        L[h] += pr[u];
       }
-      L[h] = fmaf(L[h], corr, groups16_sum(ps));
       m[h] = m_new;
 #pragma unroll
       for (int i = 0; i < NC; i++) {
@@ -229,75 +242,87 @@ __device__ void window_step(const WindowArgs &a, int nranges, int qgroups, int b
       }
     }
   }
-  // the wavefront's four groups of lanes, then the wavefronts through LDS
+  const int group = 4 * wv + g16;
 #pragma unroll
   for (int h = 0; h < QB; h++) {
 #pragma unroll
-    for (int i = 0; i < NC; i++) {
-      float4 t = o[h][i];
-      t.x += __shfl_xor(t.x, 16, 64), t.y += __shfl_xor(t.y, 16, 64), t.z += __shfl_xor(t.z, 16, 64), t.w += __shfl_xor(t.w, 16, 64);
-      t.x += __shfl_xor(t.x, 32, 64), t.y += __shfl_xor(t.y, 32, 64), t.z += __shfl_xor(t.z, 32, 64), t.w += __shfl_xor(t.w, 32, 64);
-      if (g16 == 0) *(float4 *)&S.o[wv][h][4 * (l + 16 * i)] = t;
-    }
-    if (lane == 0) S.m[wv][h] = m[h], S.l[wv][h] = L[h];
+    for (int i = 0; i < NC; i++) *(float4 *)&S.o[group][h][4 * (l + 16 * i)] = o[h][i];
+    if (l == 0) S.m[group][h] = m[h], S.l[group][h] = L[h];
   }
   __syncthreads();
   const int og = QW + KW + VW;  // the gate in the projection row
-  auto put = [&](int h, int c, float v) {
+  auto put = [&](int h, int c, float2 v, float den) {
     const int e = (h0 + h) * DV + c;
-    v *= a.out_scale;
-    out[e] = a.gated ? v * ct_sigmoid(a.p[og + e]) : v;
+    const float f = a.out_scale / den;
+    float2 y = make_float2(v.x * f, v.y * f);
+    if (a.gated) {
+      const float2 z = *(const float2 *)(a.p + og + e);
+      y.x *= ct_sigmoid(z.x), y.y *= ct_sigmoid(z.y);
+    }
+    *(float2 *)(out + e) = y;
   };
-  for (int it = tid; it < nq * DV; it += 256) {
-    const int h = it / DV, c = it - h * DV;
-    const float M = fmaxf(fmaxf(S.m[0][h], S.m[1][h]), fmaxf(S.m[2][h], S.m[3][h]));
-    const float Mu = M == -INFINITY ? 0.0f : M;
-    float v = 0.0f, den = 0.0f;
+  for (int it = tid; it < QB * DP / 2; it += 256) {
+    const int h = it / (DP / 2), c = 2 * (it % (DP / 2));
+    if (h >= nq || c >= DV) continue;
+    float M = S.m[0][h];
 #pragma unroll
-    for (int w = 0; w < 4; w++) {
+    for (int w = 1; w < 16; w++) M = fmaxf(M, S.m[w][h]);
+    const float Mu = M == -INFINITY ? 0.0f : M;
+    float2 v = make_float2(0.f, 0.f);
+    float den = 0.0f;
+#pragma unroll
+    for (int w = 0; w < 16; w++) {
       const float e = ct_exp(S.m[w][h] - Mu);
-      v = fmaf(e, S.o[w][h][c], v);
+      const float2 t = *(const float2 *)&S.o[w][h][c];
+      v.x = fmaf(e, t.x, v.x), v.y = fmaf(e, t.y, v.y);
       den = fmaf(e, S.l[w][h], den);
     }
     if (nr == 1) {
       if (a.sink) {
         const float sk = a.sink[h0 + h], top = fmaxf(M, sk), cr = ct_exp(M - top);
-        put(h, c, v * cr / fmaf(den, cr, ct_exp(sk - top)));
-      } else {
-        put(h, c, v / den);
+        v.x *= cr, v.y *= cr;
+        den = fmaf(den, cr, ct_exp(sk - top));
       }
+      put(h, c, v, den);
     } else {
-      float *rec = part + ((int64_t)(hg * nranges + range) * QB + h) * part_pitch(DV);
-      agent_store(rec + c, v);
-      if (c == 0) agent_store(rec + DV, M), agent_store(rec + DV + 1, den);
+      float *rec = part + ((int64_t)(hg * sh.ranges + range) * QB + h) * part_pitch(DV);
+      agent_store2(rec + c, v);
+      if (c == 0) agent_store2(rec + DV, make_float2(M, den));
     }
   }
   if (nr == 1) return;
   if (!last_ticket(count + hg, nr, &S.ticket)) return;
-  for (int it = tid; it < nq * DV; it += 256) {
-    const int h = it / DV, c = it - h * DV;
-    const float *rec = part + ((int64_t)hg * nranges * QB + h) * part_pitch(DV);
-    const int64_t pitch = (int64_t)QB * part_pitch(DV);
-    float mv[kWindowMaxRanges], lv[kWindowMaxRanges], ov[kWindowMaxRanges];
+  auto merge = [&](auto width) {  // up to N records, all of them requested before the first is used
+    constexpr int N = decltype(width)::value;
+    for (int it = tid; it < QB * DP / 2; it += 256) {
+      const int h = it / (DP / 2), c = 2 * (it % (DP / 2));
+      if (h >= nq || c >= DV) continue;
+      const float *rec = part + ((int64_t)hg * sh.ranges * QB + h) * part_pitch(DV);
+      const int64_t pitch = (int64_t)QB * part_pitch(DV);
+      float2 ml[N], ov[N];
 #pragma unroll
-    for (int r = 0; r < kWindowMaxRanges; r++) {  // all of them requested before the first is used
-      const float *t = rec + min(r, nr - 1) * pitch;
-      mv[r] = agent_load(t + DV), lv[r] = agent_load(t + DV + 1), ov[r] = agent_load(t + c);
-    }
-    float M = a.sink ? a.sink[h0 + h] : -INFINITY;
-#pragma unroll
-    for (int r = 0; r < kWindowMaxRanges; r++)
-      if (r < nr) M = fmaxf(M, mv[r]);
-    float v = 0.0f, den = a.sink ? ct_exp(a.sink[h0 + h] - M) : 0.0f;
-#pragma unroll
-    for (int r = 0; r < kWindowMaxRanges; r++)
-      if (r < nr) {
-        const float e = ct_exp(mv[r] - M);
-        v = fmaf(e, ov[r], v);
-        den = fmaf(e, lv[r], den);
+      for (int r = 0; r < N; r++) {
+        const float *t = rec + min(r, nr - 1) * pitch;
+        ml[r] = agent_load2(t + DV), ov[r] = agent_load2(t + c);
       }
-    put(h, c, v / den);
-  }
+      float M = a.sink ? a.sink[h0 + h] : -INFINITY;
+#pragma unroll
+      for (int r = 0; r < N; r++) M = fmaxf(M, ml[r].x);  // (the last one again and again)
+      float2 v = make_float2(0.f, 0.f);
+      float den = a.sink ? ct_exp(a.sink[h0 + h] - M) : 0.0f;
+#pragma unroll
+      for (int r = 0; r < N; r++)
+        if (r < nr) {
+          const float e = ct_exp(ml[r].x - M);
+          v.x = fmaf(e, ov[r].x, v.x), v.y = fmaf(e, ov[r].y, v.y);
+          den = fmaf(e, ml[r].y, den);
+        }
+      put(h, c, v, den);
+    }
+  };
+  if (nr <= 4) merge(std::integral_constant<int, 4>{});
+  else if (nr <= 16) merge(std::integral_constant<int, 16>{});
+  else merge(std::integral_constant<int, kWindowMaxRanges>{});
 }
 
 template <int NC>
@@ -334,71 +359,81 @@ __device__ void lightning_step(const LightningArgs &a, int block, int nblocks, f
   }
   o = row16_sum(o);
   if (l == 0) agent_store(raw + h * DV + c, o);
-  const float ss = wave_sum(l == 0 ? o * o : 0.0f);
-  if (lane == 0) red[wv] = ss;
-  __syncthreads();
-  if (tid == 0) agent_store(raw + W + block, (red[0] + red[1]) + (red[2] + red[3]));
   if (!last_ticket(count, nblocks, ticket)) return;
-  constexpr int AHEAD = 8;
-  float x[AHEAD], w[AHEAD], z[AHEAD];
+  constexpr int AHEAD = 4;  // pairs of outputs
+  float2 x[AHEAD], w[AHEAD], z[AHEAD];
   auto request = [&](int e0) {
 #pragma unroll
     for (int b = 0; b < AHEAD; b++) {
-      const int e = min(e0 + 256 * b, W - 1);
-      x[b] = agent_load(raw + e), w[b] = a.norm[e], z[b] = pg[e];
+      const int e = min(e0 + 512 * b, W - 2);
+      x[b] = agent_load2(raw + e), w[b] = *(const float2 *)(a.norm + e), z[b] = *(const float2 *)(pg + e);
     }
   };
-  request(tid);
   float t = 0.0f;
-  for (int e = tid; e < nblocks; e += 256) t += agent_load(raw + W + e);
-  t = wave_sum(t);
-  if (lane == 0) red[4 + wv] = t;
-  __syncthreads();
-  const float rstd = a.out_scale / sqrtf(((red[4] + red[5]) + (red[6] + red[7])) / (float)(a.H * a.dv) + a.eps);
-  for (int e0 = tid; e0 < W; e0 += 256 * AHEAD) {
-    if (e0 != tid) request(e0);
+  for (int e0 = 2 * tid + ((W - 1) / (512 * AHEAD)) * (512 * AHEAD); e0 >= 0; e0 -= 512 * AHEAD) {  // (the first ones last: they stay in registers)
+    request(e0);
 #pragma unroll
     for (int b = 0; b < AHEAD; b++)
-      if (e0 + 256 * b < W) out[e0 + 256 * b] = x[b] * rstd * w[b] * ct_sigmoid(z[b]);
+      if (e0 + 512 * b < W) t = fmaf(x[b].x, x[b].x, fmaf(x[b].y, x[b].y, t));
+  }
+  t = wave_sum(t);
+  if (lane == 0) red[wv] = t;
+  __syncthreads();
+  const float rstd = a.out_scale / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)(a.H * a.dv) + a.eps);
+  for (int e0 = 2 * tid; e0 < W; e0 += 512 * AHEAD) {
+    if (e0 != 2 * tid) request(e0);
+#pragma unroll
+    for (int b = 0; b < AHEAD; b++)
+      if (e0 + 512 * b < W)
+        *(float2 *)(out + e0 + 512 * b) = make_float2(x[b].x * rstd * w[b].x * ct_sigmoid(z[b].x), x[b].y * rstd * w[b].y * ct_sigmoid(z[b].y));
   }
 }
 
+// grid.x: workgroups of a key range; grid.y: the ranges, then as many rows as the lightning workgroups fill
 template <int NC, int QB>
-__global__ __launch_bounds__(256) void k_parallel_step(WindowArgs w, int ranges, int qgroups, int wblocks, float *__restrict__ wout, LightningArgs n,
-                                                       int nblocks, float *__restrict__ nout, ParallelWork k, const int *__restrict__ tokpos,
+__global__ __launch_bounds__(256) void k_parallel_step(WindowArgs w, WindowShape sh, float *__restrict__ wout, LightningArgs n, int nblocks,
+                                                       float *__restrict__ nout, ParallelWork k, const int *__restrict__ tokpos,
                                                        const int *__restrict__ ctrl) {
   __shared__ __align__(16) StepLds<NC, QB> S;
-  if ((int)blockIdx.x < wblocks) window_step<NC, QB>(w, ranges, qgroups, blockIdx.x, k.part, k.count + 1, wout, tokpos, S);
-  else lightning_step<NC>(n, blockIdx.x - wblocks, nblocks, k.raw, k.count, nout, tokpos, ctrl, S.red, &S.ticket);
+  if ((int)blockIdx.y < sh.ranges) {
+    window_step<NC, QB>(w, sh, blockIdx.x, blockIdx.y, k.part, k.count + 1, wout, tokpos, S);
+  } else {
+    const int block = ((int)blockIdx.y - sh.ranges) * (int)gridDim.x + (int)blockIdx.x;
+    if (block >= nblocks) return;
+    if (n.DK <= 64) lightning_step<1>(n, block, nblocks, k.raw, k.count, nout, tokpos, ctrl, S.red, &S.ticket);
+    else if (n.DK <= 128) lightning_step<2>(n, block, nblocks, k.raw, k.count, nout, tokpos, ctrl, S.red, &S.ticket);
+    else lightning_step<4>(n, block, nblocks, k.raw, k.count, nout, tokpos, ctrl, S.red, &S.ticket);
+  }
 }
 
 int launch_parallel_step(const WindowArgs *w, float *wout, const LightningArgs *l, float *lout, const ParallelWork &work, const int *tokpos,
                          const int *ctrl) {
   WindowArgs wa = {};
   LightningArgs la = {};
-  WindowShape sh = {0, 1, 0};
-  int nblocks = 0, qb = 1, most = 0;
+  WindowShape sh = {};
+  int nblocks = 0, pieces = 1, qb = 1;
   if (w) {
     wa = *w;
     sh = window_shape(wa);
-    qb = window_qb(wa.H / wa.G);
-    most = wa.DK > wa.DV ? wa.DK : wa.DV;
+    pieces = window_pieces(wa);
+    qb = window_qb(wa);
   }
   if (l) {
     la = *l;
     nblocks = la.H * la.DV / 16;
-    if (la.DK > most) most = la.DK;
   }
-  if (most > 256) return fail(CTHIP_E_UNSUPPORTED, "window / lightning attention: heads of %d (at most 256)", most);
-  const dim3 grid((unsigned)(sh.blocks + nblocks)), b256(256);
-#define GO(N, Q) hipLaunchKernelGGL((k_parallel_step<N, Q>), grid, b256, 0, state().stream, wa, sh.ranges, sh.qgroups, sh.blocks, wout, la, nblocks, lout, work, tokpos, ctrl)
+  if (pieces > 4 || la.DK > 256) return fail(CTHIP_E_UNSUPPORTED, "window / lightning attention: heads of more than 256");
+  const int gx = w ? sh.heads : nblocks;
+  const dim3 grid((unsigned)gx, (unsigned)(sh.ranges + (nblocks + gx - 1) / gx)), b256(256);
+#define GO(N, Q) hipLaunchKernelGGL((k_parallel_step<N, Q>), grid, b256, 0, state().stream, wa, sh, wout, la, nblocks, lout, work, tokpos, ctrl)
 #define GO_N(N)            \
   if (qb <= 1) GO(N, 1);   \
   else if (qb <= 2) GO(N, 2); \
   else GO(N, 4)
-  if (most <= 64) { GO_N(1); }
-  else if (most <= 128) { GO_N(2); }
-  else { GO_N(4); }
+  if (pieces <= 1) { GO_N(1); }
+  else if (pieces <= 2) { GO_N(2); }
+  else if (qb <= 1) GO(4, 1);
+  else GO(4, 2);
 #undef GO_N
 #undef GO
   CTHIP_LAUNCH_CHECK();
