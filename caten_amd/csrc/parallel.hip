@@ -3,9 +3,9 @@
 //
 //   window     workgroup (key range, key/value head, up to QB of its query heads).  It takes the root mean squares of all
 //              queries and keys, normalises and rotates its own, and attends over its share of the ring: 16 lanes per row,
-//              16 rows a tile, range r takes the r-th run of `2^lper` tiles.  Rings are walked by row, not by position, so the
-//              first rows are asked for before the position is known; which position a row holds follows from it.  The new
-//              key and value come from the projection row; the range that owns their row of the ring stores them.  While
+//              16 rows a tile, range r takes the r-th run of `2^lper` tiles.  Rings are walked by row, not by position; which
+//              position a row holds follows from the step's.  The new key and value come from the projection row; the range
+//              that owns their row of the ring stores them.  While
 //              few rows are held, few ranges have any, and a single one finishes by itself.  Every group of 16 lanes keeps a
 //              softmax of its own; they meet in LDS.
 //   lightning  workgroup (head, 16 value columns), 16 lanes per column: the state's rows are read once, updated, read out
@@ -125,6 +125,9 @@ __device__ void window_step(const WindowArgs &a, const WindowShape &sh, int hg, 
     }
   };
   const int first = range << sh.lper;
+  const int held = min(pos + 1, rows), tiles = (held + 15) >> 4, nr = ((tiles - 1) >> sh.lper) + 1;
+  if (range >= nr) return;  // no row of this range yet (uniform)
+  const int end = min(first + (1 << sh.lper), tiles);
 #pragma unroll
   for (int u = 0; u < U; u++) request(u, first + u);
   float qs = 1.0f, ks = 1.0f;
@@ -138,9 +141,6 @@ __device__ void window_step(const WindowArgs &a, const WindowShape &sh, int hg, 
     sq = wave_sum(sq), sk = wave_sum(sk);
     if (lane == 0) S.red[wv] = sq, S.red[4 + wv] = sk;
   }
-  const int held = min(pos + 1, rows), tiles = (held + 15) >> 4, nr = ((tiles - 1) >> sh.lper) + 1;
-  if (range >= nr) return;  // (uniform)
-  const int end = min(first + (1 << sh.lper), tiles);
   float2 qc[QE], kc = make_float2(1.0f, 0.0f);
   auto angle = [&](int d) { return d < 2 * half ? a.rope[(int64_t)pos * half + (d < half ? d : d - half)] : make_float2(1.0f, 0.0f); };
 #pragma unroll
