@@ -132,7 +132,9 @@ def zuselix(config, tensors, tokens):
 def yarn(rot):
     """rotation frequencies (dims / 2) and the factor of cosine and sine: slow rotations are stretched by `factor`, fast
     ones are left, a linear ramp over the pair index lies between"""
-    dims, base, sc = rot["dims"], rot["base"], rot["scaling"]
+    dims, base, sc = rot["dims"], rot["base"], rot.get("scaling")
+    if sc is None:
+        return base ** (-2.0 * np.arange(dims // 2) / dims), 1.0
 
     def pair_that_turns(times):  # the (real-valued) pair that turns `times` times over the original context
         return dims * np.log(sc["original"] / (2 * np.pi * times)) / (2 * np.log(base))
@@ -153,21 +155,24 @@ def rotate_half(x, positions, freqs, mscale):
     return np.concatenate([u * c - v * s, v * c + u * s, x[..., 2 * n:]], -1)
 
 
-def window_attention(h, m, w, eps):
-    """grouped-query attention over the last mask.size positions; the softmax has a sink of score 0"""
+def window_attention(h, m, w, eps, bias=True, qk_norm=True, sink=0.0, gate=True):
+    """grouped-query attention over the last mask.size positions; sink: a score per head or for all of them (-inf = none)"""
     T, H, G, dk, dv = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    freqs, mscale = yarn(m["rot"])
-    q = rms_norm(h @ w("q").T + w("q.b"), w("q.norm"), eps).reshape(T, H, dk)
-    k = rms_norm(h @ w("k").T + w("k.b"), w("k.norm"), eps).reshape(T, G, dk)
-    v = (h @ w("v").T + w("v.b")).reshape(T, G, dv)
-    q, k = rotate_half(q, range(T), freqs, mscale), rotate_half(k, range(T), freqs, mscale)
+    q, k, v = (h @ w(n).T + (w(n + ".b") if bias else 0.0) for n in ("q", "k", "v"))
+    if qk_norm:
+        q, k = rms_norm(q, w("q.norm"), eps), rms_norm(k, w("k.norm"), eps)
+    q, k, v = q.reshape(T, H, dk), k.reshape(T, G, dk), v.reshape(T, G, dv)
+    if m["rot"] is not None:
+        freqs, mscale = yarn(m["rot"])
+        q, k = rotate_half(q, range(T), freqs, mscale), rotate_half(k, range(T), freqs, mscale)
     back = np.arange(T)[:, None] - np.arange(T)[None, :]
     hidden = np.where((back >= 0) & (back < m["mask"]["size"]), 0.0, -np.inf)
+    sink = np.broadcast_to(sink, (H,))
     o = np.zeros((T, H, dv))
     for n in range(H):
         g = n // (H // G)
-        o[:, n] = sink_softmax(q[:, n] @ k[:, g].T * m["scale"] + hidden, 0.0) @ v[:, g]
-    return (o.reshape(T, -1) * sigmoid(h @ w("g").T)) @ w("o").T
+        o[:, n] = sink_softmax(q[:, n] @ k[:, g].T * m["scale"] + hidden, sink[n]) @ v[:, g]
+    return (o.reshape(T, -1) * (sigmoid(h @ w("g").T) if gate else 1.0)) @ w("o").T
 
 
 def lightning_recurrence(q, k, v, decay):

@@ -75,6 +75,76 @@ def test_norms_positions_and_gates():
                                       np.sin(3 / 10000 ** (2 / 3)), np.cos(3 / 10000 ** (2 / 3))], atol=1e-12)
 
 
+def test_rotation_is_a_complex_product():
+    rng = np.random.default_rng(6)
+    x, f = rng.standard_normal((5, 3, 10)), np.array([1.0, 0.3, 0.01, 2.5])
+    pos = [0, 1, 7, 100, 4000]
+    z = (x[..., :4] + 1j * x[..., 4:8]) * 1.2 * np.exp(1j * np.asarray(pos)[:, None, None] * f)
+    got = mixers.rotate_half(x, pos, f, 1.2)
+    np.testing.assert_allclose(got, np.concatenate([z.real, z.imag, x[..., 8:]], -1), atol=1e-9)
+
+
+def test_yarn_frequencies():
+    plain = 100.0 ** (-np.arange(0, 16, 2) / 16)
+    f, m = mixers.yarn(dict(dims=16, base=100.0))
+    assert m == 1.0
+    np.testing.assert_allclose(f, plain, rtol=1e-14)
+    f, m = mixers.yarn(dict(dims=16, base=100.0, scaling=dict(factor=1.0, original=64, fast=8.0, slow=1.0)))
+    assert m == 1.0
+    np.testing.assert_allclose(f, plain, rtol=1e-14)
+    # pair i turns original f_i / (2 pi) times: above `fast` turns it stays, below `slow` it is divided by the factor
+    f, m = mixers.yarn(dict(dims=64, base=1e4, scaling=dict(factor=4.0, original=2048, fast=32.0, slow=1.0)))
+    plain = 1e4 ** (-np.arange(0, 64, 2) / 64)
+    turns = 2048 * plain / (2 * np.pi)
+    assert m == pytest.approx(0.1 * np.log(4.0) + 1.0)
+    quotient = plain / f
+    assert np.all(quotient[turns > 45] == 1.0) and np.allclose(quotient[turns < 0.7], 4.0) and np.all(np.diff(quotient) >= -1e-12)
+    # the ramp is clipped at the first pair and at the last entry of the head, and may have no width
+    f, _ = mixers.yarn(dict(dims=8, base=10.0, scaling=dict(factor=2.0, original=1, fast=100.0, slow=50.0)))
+    np.testing.assert_allclose(f, np.r_[1.0, 10.0 ** (-np.arange(2, 8, 2) / 8) / 2], rtol=1e-14)
+
+
+def test_window_attention_against_masked_softmax():
+    """grouped heads, window and zero sink as one dense softmax with a column of zeros"""
+    rng = np.random.default_rng(7)
+    T, m = 20, mm.window(6, 2, 8, 5, 7, 0.4, 6)
+    cfg = mm.matalix([mm.parallel(m, mm.lightning(1, 4, 4))], width=24)
+    w = {k[12:]: v.astype(np.float64) for k, v in mm.weights(cfg, 3).items() if k.startswith("l0.mix.left.")}
+    h = rng.standard_normal((T, 24))
+    got = mixers.window_attention(h, m, w.__getitem__, 1e-5)
+    t = {k: torch.tensor(v) for k, v in w.items()}
+    x = torch.tensor(h)
+    q = F.rms_norm(F.linear(x, t["q"], t["q.b"]), (48,), t["q.norm"], 1e-5).view(T, 6, 8)
+    k = F.rms_norm(F.linear(x, t["k"], t["k.b"]), (16,), t["k.norm"], 1e-5).view(T, 2, 8)
+    v = F.linear(x, t["v"], t["v.b"]).view(T, 2, 5)
+    f, c = mixers.yarn(m["rot"])
+    q, k = (torch.tensor(mixers.rotate_half(a.numpy(), range(T), f, c)) for a in (q, k))
+    k, v = k.repeat_interleave(3, 1), v.repeat_interleave(3, 1)
+    s = torch.einsum("ihd,jhd->hij", q, k) * 0.4
+    seen = torch.ones(T, T, dtype=torch.bool).tril() & torch.ones(T, T, dtype=torch.bool).triu(-6)
+    s = torch.cat([s.masked_fill(~seen, -torch.inf), torch.zeros(6, T, 1, dtype=torch.float64)], -1)
+    o = torch.einsum("hij,jhd->ihd", s.softmax(-1)[..., :-1], v).reshape(T, -1) * torch.sigmoid(x @ t["g"].T)
+    np.testing.assert_allclose(got, (o @ t["o"].T).numpy(), atol=1e-11)
+
+
+def test_lightning_recurrence_against_its_quadratic_form():
+    rng = np.random.default_rng(8)
+    q, k, v = (rng.standard_normal((30, n)) for n in (6, 6, 4))
+    for g in (0.0, 0.7, 1.0):
+        back = np.arange(30)[:, None] - np.arange(30)[None, :]
+        D = np.where(back >= 0, np.float64(g) ** np.maximum(back, 0), 0.0)
+        o, S = mixers.lightning_recurrence(q, k, v, g)
+        np.testing.assert_allclose(o, (D * (q @ k.T)) @ v, atol=1e-11)
+        np.testing.assert_allclose(S, (k * D[-1][:, None]).T @ v, atol=1e-11)
+
+
+def test_clamped_unit():
+    w = {"gate": np.array([[1.0], [1.0]]), "up": np.array([[1.0], [-1.0]]), "down": np.eye(2)}
+    g = np.minimum([[5.0], [-9.0]], 2.0)
+    u = np.clip(np.array([[5.0, -5.0], [-9.0, 9.0]]), -2.0, 2.0)
+    np.testing.assert_allclose(mixers.clamped_mlp(np.array([[5.0], [-9.0]]), 2.0, w.__getitem__), g * mixers.sigmoid(1.702 * g) * (u + 1))
+
+
 # ---- model directories ----
 def test_safetensors_round_trip(tmp_path):
     p = str(tmp_path / "m.safetensors")
@@ -140,6 +210,49 @@ def test_configuration():
         llm.zuselix_config(bad)
 
 
+def test_configuration_of_parallel_mixers():
+    cfg = mm.matalix([mm.parallel(mm.window(6, 3, 10, 12, 9, 0.3, 8), mm.lightning(2, 7, 5, [0.5, 0.25]), 0.1, 0.2, ff=40, limit=1.5), mm.parallel()],
+                     width=30, vocab=50, eps=1e-3, loop=dict(start=0, stop=1, times=3))
+    c = llm.matalix_config(cfg)
+    assert (c["dim"], c["vocab"], c["eps"], c["norm"], c["norm_plus_one"], c["tied_head"], c["loop"]) == (30, 50, 1e-3, "rmsnorm", True, True, (0, 1, 3))
+    left, right = c["layers"][0]["mixers"]
+    assert left == dict(mixer="window", heads=6, kv_heads=3, dim=10, vdim=12, scale=0.3, window=9, bias=True, qk_norm=True, sink="zero", gate=True,
+                        out_scale=0.1, rot=dict(dims=8, base=10000.0, factor=8.0, original=64, fast=8.0, slow=1.0))
+    assert right == dict(mixer="lightning", heads=2, dim=7, vdim=5, decay=[0.5, 0.25], out_scale=0.2)
+    assert (c["layers"][0]["ffn"], c["layers"][0]["glu"], c["layers"][0]["layer_scale"]) == (40, (1.702, 1.5, 1.0), True)
+    assert "ffn" not in c["layers"][1]
+    del cfg["loop"]
+    assert llm.matalix_config(cfg)["loop"] is None
+    bad = mm.matalix([mm.delta()])
+    with pytest.raises(ValueError, match="layer 0: mixer type 'delta'"):
+        llm.matalix_config(bad)
+    bad = mm.matalix([mm.parallel(ff=8)])
+    bad["layers"][0]["mlp"]["kind"] = "experts"
+    with pytest.raises(ValueError, match="kind 'experts'"):
+        llm.matalix_config(bad)
+
+
+def test_looped_layers_of_the_restatement():
+    """a loop is its layers written out, with the embedding added in between"""
+    layers = [mm.parallel(ff=8), mm.parallel(mm.window(2, 1, 8, 8, 5)), mm.parallel()]
+    cfg = mm.matalix(layers, width=16, vocab=20, loop=dict(start=1, stop=3, times=2))
+    w, toks = mm.weights(cfg, 4), mm.tokens(cfg, 12)
+    logits, stream = mixers.matalix(cfg, w, toks)
+    assert stream.shape == (5, 12, 16)
+    t = {k: v.astype(np.float64) for k, v in w.items()}
+    x0 = x = t["embed"][toks]
+    for step in (0, 1, 2, None, 1, 2):
+        if step is None:
+            x = x + x0
+            continue
+        one = dict(cfg, layers=[layers[step]], loop=None)
+        rest = {k.replace(f"l{step}.", "l0.", 1): v for k, v in t.items() if k.startswith(f"l{step}.")}
+        # the layer as a model of its own whose embedding table holds the stream
+        x = mixers.matalix(one, dict(rest, embed=x, **{"final.norm": t["final.norm"]}), range(12))[1][0]
+    np.testing.assert_allclose(stream[-1], x, atol=1e-10)
+    np.testing.assert_allclose(logits, mixers.rms_norm(x, 1 + t["final.norm"], 1e-5) @ t["embed"].T, atol=1e-9)
+
+
 def test_registry(tmp_path):
     (tmp_path / "config.json").write_text(json.dumps({"architecture": "Other"}))
     with pytest.raises(ValueError, match="'Other' is not registered .known: Matalix, Zuselix"):
@@ -153,6 +266,12 @@ def test_shapes_of_the_measured_sizes():
     for name, cfg in synth.ZUSELIX_CONFIGS.items():
         shapes = synth.zuselix_shapes(cfg)
         assert shapes["l2.mix.uk"] == (cfg["layers"][2]["mixer"]["heads"] * 128, 512) and "l0.mix.A_log" in shapes, name
+    for name, cfg in synth.MATALIX_CONFIGS.items():
+        shapes, left = synth.matalix_shapes(cfg), cfg["layers"][0]["mixer"]["left"]
+        assert shapes["l3.mix.left.q"] == shapes["l3.mix.left.o"][::-1] == (left["heads"] * 128, cfg["width"]) and "head" not in shapes, name
+    import bench_mixed
+    assert sum(bench_mixed.layer_runs(synth.MATALIX_CONFIGS["matalix-1b"])) == 22
+    assert sum(bench_mixed.layer_runs(synth.ZUSELIX_CONFIGS["zuselix-1b"])) == 21
 
 
 def test_c_abi_before_a_device_is_there():
